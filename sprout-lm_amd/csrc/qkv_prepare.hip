@@ -29,6 +29,8 @@ struct PrepareArgs {
   float magnitude;             // on every cosine and sine (1: a plain rotation)
   const float* q_mult;         // one number per query head that multiplies its turned queries (null: none)
   int head_norm;               // every q and k head, after it has turned, is divided by its root mean square over dim (eps inside)
+  int maps;                    // > 1: a key head holds this many maps of dim numbers side by side in its `width`, and of the nq
+                               // query rows row n is map n % maps of a head: its numbers stand where that map's do, zeros elsewhere
 };
 
 // Sum of the squares of n numbers over the whole block, as the scale of an RMS norm; every thread gets it.
@@ -46,12 +48,12 @@ template <typename T>
 __device__ __forceinline__ void prepare_head(const PrepareArgs& a, int t, int head, float q_scale, float k_scale, int slot,
                                              int lane, int count, float* scratch, bool whole_block) {
   const T* row = (const T*)a.proj + size_t(t) * a.stride;
-  const int nq = a.nq, nkv = a.nkv, D = a.dim, V = a.vdim, W = a.width;
+  const int nq = a.nq, nkv = a.nkv, nk = nkv * a.maps, D = a.dim, V = a.vdim, W = a.width;      // nk: rows of keys
   const int page = slot >= 0 ? slot / a.page_size : 0, off = slot >= 0 ? slot % a.page_size : 0;
-  if (head >= nq + nkv) {
+  if (head >= nq + nk) {
     // values: blended with the first flagged layer's, or kept for the later layers; written dimension-major
-    const int g = head - nq - nkv;
-    const T* vrow = row + size_t(nq + nkv) * D + size_t(g) * V;
+    const int g = head - nq - nk;
+    const T* vrow = row + size_t(nq + nk) * D + size_t(g) * V;
     const float lam = a.blend ? to_float(*(const T*)a.blend) : 0.f;
     T* first = a.first ? (T*)a.first + size_t(t) * nkv * V + size_t(g) * V : nullptr;
     for (int d = lane; d < W; d += count) {
@@ -72,7 +74,12 @@ __device__ __forceinline__ void prepare_head(const PrepareArgs& a, int t, int he
   if (nw) nw += size_t(is_q ? head : head - nq) * D;
   const float scale = is_q ? q_scale : k_scale;
   T* dst = is_q ? (T*)a.q_out + (size_t(t) * nq + head) * W
-                : (T*)a.k_pool + ((size_t(page) * nkv + (head - nq)) * a.page_size + off) * W;
+                : (T*)a.k_pool + ((size_t(page) * nkv + (head - nq) / a.maps) * a.page_size + off) * W;
+  const int map = (is_q ? head : head - nq) % a.maps, before = map * D;      // where the head's numbers begin in its width
+  dst += before;
+  const int behind = is_q || map == a.maps - 1 ? W - before : D;             // how far this row writes, zeros from D on
+  if (is_q)
+    for (int d = lane; d < before; d += count) dst[d - before] = from_float<T>(0.f);
   const int half = a.rotary_dim / 2;
   auto normed = [&](int e) {
     float x = to_float(src[e]);
@@ -90,7 +97,7 @@ __device__ __forceinline__ void prepare_head(const PrepareArgs& a, int t, int he
     unit = 1.0f / sqrtf(sq / float(D) + a.eps);
   }
   if (is_q && a.q_mult) unit *= a.q_mult[head];
-  for (int d = lane; d < W; d += count) {
+  for (int d = lane; d < behind; d += count) {
     if (d >= D) { dst[d] = from_float<T>(0.f); continue; }
     if (d >= 2 * half) { dst[d] = from_float<T>(normed(d) * unit); continue; }
     if (d >= half) continue;          // written by the owner of its pair
@@ -129,11 +136,11 @@ __device__ __forceinline__ float4 round4(float4 v) {
 __device__ __forceinline__ void prepare_head_fours(const PrepareArgs& a, int t, int head, float q_scale, float k_scale, int slot,
                                                    int lane, int count) {
   const bf16_t* row = (const bf16_t*)a.proj + size_t(t) * a.stride;
-  const int nq = a.nq, nkv = a.nkv, D = a.dim, V = a.vdim, W = a.width;
+  const int nq = a.nq, nkv = a.nkv, nk = nkv * a.maps, D = a.dim, V = a.vdim, W = a.width;
   const int page = slot >= 0 ? slot / a.page_size : 0, off = slot >= 0 ? slot % a.page_size : 0;
-  if (head >= nq + nkv) {
-    const int g = head - nq - nkv;
-    const bf16_t* vrow = row + size_t(nq + nkv) * D + size_t(g) * V;
+  if (head >= nq + nk) {
+    const int g = head - nq - nk;
+    const bf16_t* vrow = row + size_t(nq + nk) * D + size_t(g) * V;
     const float lam = a.blend ? to_float(*(const bf16_t*)a.blend) : 0.f;
     bf16_t* first = a.first ? (bf16_t*)a.first + size_t(t) * nkv * V + size_t(g) * V : nullptr;
     for (int d = 4 * lane; d < W; d += 4 * count) {
@@ -166,7 +173,12 @@ __device__ __forceinline__ void prepare_head_fours(const PrepareArgs& a, int t, 
   if (nw) nw += size_t(is_q ? head : head - nq) * D;
   const float scale = is_q ? q_scale : k_scale;
   bf16_t* dst = is_q ? (bf16_t*)a.q_out + (size_t(t) * nq + head) * W
-                     : (bf16_t*)a.k_pool + ((size_t(page) * nkv + (head - nq)) * a.page_size + off) * W;
+                     : (bf16_t*)a.k_pool + ((size_t(page) * nkv + (head - nq) / a.maps) * a.page_size + off) * W;
+  const int map = (is_q ? head : head - nq) % a.maps, before = map * D;
+  dst += before;
+  const int behind = is_q || map == a.maps - 1 ? W - before : D;
+  if (is_q)
+    for (int d = 4 * lane; d < before; d += 4 * count) *reinterpret_cast<uint2*>(dst + d - before) = make_uint2(0u, 0u);
   const int half = a.rotary_dim / 2;
   const float mult = is_q && a.q_mult ? a.q_mult[head] : 1.f;
   auto normed = [&](int e) {
@@ -177,7 +189,7 @@ __device__ __forceinline__ void prepare_head_fours(const PrepareArgs& a, int t, 
     }
     return make_float4(x.x * mult, x.y * mult, x.z * mult, x.w * mult);
   };
-  for (int d = 4 * lane; d < W; d += 4 * count) {
+  for (int d = 4 * lane; d < behind; d += 4 * count) {
     if (d >= D) { *reinterpret_cast<uint2*>(dst + d) = make_uint2(0u, 0u); continue; }
     if (d >= 2 * half) { *reinterpret_cast<uint2*>(dst + d) = pack4(normed(d)); continue; }
     if (d >= half) continue;
@@ -213,13 +225,13 @@ __global__ __launch_bounds__(256) void qkv_prepare_kernel(PrepareArgs a) {
   const int t = blockIdx.x;
   const T* row = (const T*)a.proj + size_t(t) * a.stride;
   const int slot = a.slot_mapping ? a.slot_mapping[t] : -1;
-  const int heads = a.nq + 2 * a.nkv;
+  const int heads = a.nq + (a.maps + 1) * a.nkv;
   if (PER_HEAD) {
     const int head = blockIdx.y;
     float scale = 1.f;
-    if (a.q_norm && head < a.nq + a.nkv && (head < a.nq || slot >= 0)) {
+    if (a.q_norm && head < a.nq + a.nkv * a.maps && (head < a.nq || slot >= 0)) {
       const T* whole = head < a.nq ? row : row + size_t(a.nq) * a.dim;
-      const int n = (head < a.nq ? a.nq : a.nkv) * a.dim;
+      const int n = (head < a.nq ? a.nq : a.nkv * a.maps) * a.dim;
       if constexpr (FOURS) scale = row_scale_fours(whole, n, a.eps, scratch);
       else scale = row_scale(whole, n, a.eps, scratch);
     }
@@ -231,10 +243,10 @@ __global__ __launch_bounds__(256) void qkv_prepare_kernel(PrepareArgs a) {
   if (a.q_norm) {
     if constexpr (FOURS) {
       q_scale = row_scale_fours(row, a.nq * a.dim, a.eps, scratch);
-      k_scale = row_scale_fours(row + size_t(a.nq) * a.dim, a.nkv * a.dim, a.eps, scratch);
+      k_scale = row_scale_fours(row + size_t(a.nq) * a.dim, a.nkv * a.maps * a.dim, a.eps, scratch);
     } else {
       q_scale = row_scale(row, a.nq * a.dim, a.eps, scratch);
-      k_scale = row_scale(row + size_t(a.nq) * a.dim, a.nkv * a.dim, a.eps, scratch);
+      k_scale = row_scale(row + size_t(a.nq) * a.dim, a.nkv * a.maps * a.dim, a.eps, scratch);
     }
   }
   const int wave = threadIdx.x >> 6, waves = blockDim.x >> 6;
@@ -244,19 +256,67 @@ __global__ __launch_bounds__(256) void qkv_prepare_kernel(PrepareArgs a) {
   }
 }
 
+// The difference of two maps' outputs, normed: out[t, h, :V] = (o / sqrt(mean(o^2) + eps)) * factor with
+// o = maps[t, 2 h] - lambda * maps[t, 2 h + 1], each map V of `width` numbers.  A wave per (token, head), its numbers in
+// registers (PER a lane) between the sum of squares and the store.
+template <typename TI, typename T, int PER>
+__global__ __launch_bounds__(256) void map_difference_kernel(const TI* __restrict__ maps, const float* __restrict__ lambda,
+                                                             float eps, float factor, T* __restrict__ out, int rows, int V, int width) {
+  const int row = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (row >= rows) return;
+  const float lam = *lambda;
+  const TI *a = maps + size_t(2) * row * width, *b = a + width;
+  float o[PER], sq = 0.f;
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int d = lane + 64 * i;
+    o[i] = d < V ? to_float(a[d]) - lam * to_float(b[d]) : 0.f;
+    sq = fmaf(o[i], o[i], sq);
+  }
+  const float unit = factor / sqrtf(wave_sum(sq) / float(V) + eps);
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int d = lane + 64 * i;
+    if (d < V) out[size_t(row) * V + d] = from_float<T>(o[i] * unit);
+  }
+}
+
 }  // namespace sprout
 
 using namespace sprout;
+
+extern "C" int sp_map_difference(void* stream, int in_dtype, const void* maps, int width, const float* lambda, float eps,
+                                 float factor, int dtype, void* out, int T, int heads, int vdim) {
+  SP_REQUIRE(T >= 0 && heads > 0 && vdim > 0 && vdim <= 512 && width >= vdim && maps && lambda && out, "sp_map_difference: bad arguments");
+  SP_REQUIRE((in_dtype == kF32 || in_dtype == kBF16) && (dtype == kF32 || dtype == kBF16), "sp_map_difference: unsupported dtypes");
+  if (T == 0) return 0;
+  const int rows = T * heads;
+  hipStream_t s = (hipStream_t)stream;
+#define SP_DIFF(TI, TT, PER) map_difference_kernel<TI, TT, PER><<<(rows + 3) / 4, 256, 0, s>>>((const TI*)maps, lambda, eps, factor, (TT*)out, rows, vdim, width)
+#define SP_DIFF_TYPES(PER)                                                       \
+  do {                                                                           \
+    if (in_dtype == kF32 && dtype == kF32) SP_DIFF(float, float, PER);           \
+    else if (in_dtype == kF32) SP_DIFF(float, bf16_t, PER);                      \
+    else if (dtype == kF32) SP_DIFF(bf16_t, float, PER);                         \
+    else SP_DIFF(bf16_t, bf16_t, PER);                                           \
+  } while (0)
+  if (vdim <= 128) SP_DIFF_TYPES(2);
+  else if (vdim <= 256) SP_DIFF_TYPES(4);
+  else SP_DIFF_TYPES(8);
+#undef SP_DIFF_TYPES
+#undef SP_DIFF
+  return check_launch("sp_map_difference");
+}
 
 extern "C" int sp_qkv_prepare(void* stream, int dtype, const void* proj, long long stride, int nq, int nkv, int dim, int vdim,
                               int width, const void* q_norm, const void* k_norm, float eps, const int32_t* positions,
                               const float* inv_freq, const float* inv_freq_tail, int rotary_dim, const void* blend,
                               void* first, int keep_first, const int32_t* slot_mapping, void* k_pool, void* v_pool,
                               int page_size, int num_pages, void* q_out, int T, float magnitude, int head_norm,
-                              const float* q_mult) {
-  SP_REQUIRE(T >= 0 && nq > 0 && nkv > 0 && dim > 0 && vdim > 0 && width >= dim && width >= vdim,
+                              const float* q_mult, int maps) {
+  SP_REQUIRE(T >= 0 && nq > 0 && nkv > 0 && dim > 0 && vdim > 0 && maps > 0 && nq % maps == 0 && width >= maps * dim && width >= vdim,
              "sp_qkv_prepare: bad sizes nq=%d nkv=%d dim=%d vdim=%d width=%d", nq, nkv, dim, vdim, width);
-  SP_REQUIRE(stride >= (long long)(nq + nkv) * dim + (long long)nkv * vdim, "sp_qkv_prepare: a row of %lld numbers does not hold q, k and v", stride);
+  SP_REQUIRE(stride >= (long long)(nq + nkv * maps) * dim + (long long)nkv * vdim, "sp_qkv_prepare: a row of %lld numbers does not hold q, k and v", stride);
   SP_REQUIRE(proj && q_out, "sp_qkv_prepare: null operand");
   SP_REQUIRE((q_norm == nullptr) == (k_norm == nullptr), "sp_qkv_prepare: queries and keys are normed together or not at all");
   SP_REQUIRE(rotary_dim >= 0 && rotary_dim % 2 == 0 && rotary_dim <= dim, "sp_qkv_prepare: %d numbers cannot turn in a head of %d", rotary_dim, dim);
@@ -265,16 +325,16 @@ extern "C" int sp_qkv_prepare(void* stream, int dtype, const void* proj, long lo
   SP_REQUIRE(!slot_mapping || (k_pool && v_pool && page_size > 0 && num_pages > 0), "sp_qkv_prepare: bad cache geometry");
   if (T == 0) return 0;
   PrepareArgs a = {proj, stride, nq, nkv, dim, vdim, width, q_norm, k_norm, eps, positions, inv_freq, inv_freq_tail, rotary_dim,
-                   blend, first, keep_first, slot_mapping, k_pool, v_pool, page_size, q_out, magnitude, q_mult, head_norm};
+                   blend, first, keep_first, slot_mapping, k_pool, v_pool, page_size, q_out, magnitude, q_mult, head_norm, maps};
   hipStream_t s = (hipStream_t)stream;
-  SP_REQUIRE(nq + 2 * nkv <= 65535, "sp_qkv_prepare: %d heads are more than a launch's second dimension holds", nq + 2 * nkv);
+  SP_REQUIRE(nq + (maps + 1) * nkv <= 65535, "sp_qkv_prepare: %d heads are more than a launch's second dimension holds", nq + (maps + 1) * nkv);
   SP_REQUIRE(dtype == kF32 || dtype == kBF16, "sp_qkv_prepare: unsupported dtype %d", dtype);
   auto eight = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 7) == 0; };
   const bool fours = dtype == kBF16 && !inv_freq_tail && !head_norm && magnitude == 1.0f && dim % 4 == 0 && vdim % 4 == 0 && width % 4 == 0 && rotary_dim % 8 == 0 &&
                      stride % 4 == 0 && eight(proj) && eight(q_out) && eight(q_norm) && eight(k_norm) && eight(first) &&
                      eight(k_pool);
-  if (T * (nq + 2 * nkv) <= 2048) {      // few tokens: a block per head
-    const dim3 grid(T, nq + 2 * nkv);
+  if (T * (nq + (maps + 1) * nkv) <= 2048) {      // few tokens: a block per head
+    const dim3 grid(T, nq + (maps + 1) * nkv);
     const int threads = width <= 64 ? 64 : 128;
     if (dtype == kF32) qkv_prepare_kernel<float, true, false><<<grid, threads, 0, s>>>(a);
     else if (fours) qkv_prepare_kernel<bf16_t, true, true><<<grid, 64, 0, s>>>(a);

@@ -146,8 +146,15 @@ int sp_qkv_prepare(void* stream, int dtype, const void* proj, long long stride, 
                    const void* q_norm, const void* k_norm, float eps, const int32_t* positions, const float* inv_freq,
                    const float* inv_freq_tail, int rotary_dim, const void* blend, void* first, int keep_first,
                    const int32_t* slot_mapping, void* k_pool, void* v_pool, int page_size, int num_pages, void* q_out, int T, float magnitude,
-                   int head_norm, const float* q_mult);
-// q_mult (null: none): one float per query head that multiplies its turned queries.
+                   int head_norm, const float* q_mult, int maps);
+// q_mult (null: none): one float per query head that multiplies its turned queries.  maps: 1, or how many keys of dim numbers
+// a key head holds side by side in its width (each turns by itself; the row of proj holds nkv * maps of them, and nkv * maps *
+// dim numbers of keys), while query row n (of nq, a multiple of maps) is map n % maps of its head: its numbers stand in q_out
+// where that map's do in a key, zeros elsewhere, so that its product with a whole key is the map's own.
+// out[t, h, :vdim] = o / sqrt(mean(o^2) + eps) * factor with o = maps[t, 2 h] - *lambda * maps[t, 2 h + 1]; maps [T, 2 heads,
+// width] of in_dtype (vdim numbers each, vdim up to 512), lambda one float on the device, out [T, heads * vdim] of dtype.
+int sp_map_difference(void* stream, int in_dtype, const void* maps, int width, const float* lambda, float eps, float factor,
+                      int dtype, void* out, int T, int heads, int vdim);
 
 // dst (dst_dtype) = src (src_dtype), n elements
 
@@ -212,18 +219,20 @@ int sp_embed_bigram(void* stream, int table_dtype, const void* table, const void
                     const int32_t* state_slots, int32_t* last_token, float* residual, int T, int H, int V,
                     long long buckets, long long mul_prev, long long mul_cur);
 
-// Attention over a latent, between the input projections and the attention kernel.  A row of proj holds per head
-// [dim unrotated, rot rotated] query numbers from column q_off on, and at dkv_off the latent (rank numbers) and
-// one rotated key part (rot numbers).  Writes, per token: the RMS-normed latent and the turned key part as the key
-// [rank + rot] of the one key/value head at slot_mapping[t] (null: nothing is cached), the latent as the value
-// (the value pool's last rot columns are left alone), and every head's turned query part into
-// q_out[t, head, rank : rank + rot] (rows of heads * (rank + rot)).  The first rot_dims numbers of a rotated part
-// turn, (2i, 2i + 1) together, by positions[t] * freq[i] with cosine and sine times `magnitude`; exact != 0: the
-// angle and its cosine and sine in float64.
-int sp_latent_prepare(void* stream, int dtype, const void* proj, int proj_stride, int q_off, int heads, int dim, int rot,
-                      int dkv_off, int rank, int norm_w_dtype, const void* norm_w, float eps, const int32_t* positions,
-                      const double* freq, int rot_dims, float magnitude, int exact, const int32_t* slot_mapping,
-                      void* k_pool, void* v_pool, int page_size, int num_pages, void* q_out, int T);
+// Attention over a latent, between the input projections and the attention kernel: three jobs, each done where its rows are
+// given.  (1) kv: rows hold at kv_off the latent (rank numbers) and one rotated key part (rot numbers); the RMS-normed latent
+// and the turned key part go as the key [rank + rot, zeros up to width] of the one key/value head to slot_mapping[t]
+// (negative: not written), the latent as the value (the value pool's columns behind it are left alone).  (2) q: rows hold per
+// head [dim unrotated, rot rotated] query numbers from column q_off on; every head's turned part goes to
+// q_out[t, head, rank : rank + rot], zeros behind it (rows of heads * width).  (3) cq: rows hold at cq_off a query latent of
+// cq_rank numbers, which goes RMS-normed to cq_out [T, cq_rank].  Both norms' weights are of norm_w_dtype.  The first rot_dims
+// numbers of a rotated part turn, pairing 0: (2i, 2i + 1), 1: (i, i + rot_dims / 2) together, by positions[t] * freq[i] with
+// cosine and sine times `magnitude`; exact != 0: the angle and its cosine and sine in float64.
+int sp_latent_prepare(void* stream, int dtype, int heads, int dim, int rot, int rank, int width, int norm_w_dtype, float eps,
+                      const int32_t* positions, const double* freq, int rot_dims, float magnitude, int pairing, int exact,
+                      const void* kv, int kv_stride, int kv_off, const void* kv_norm, const int32_t* slot_mapping, void* k_pool,
+                      void* v_pool, int page_size, int num_pages, const void* q, int q_stride, int q_off, void* q_out,
+                      const void* cq, int cq_stride, int cq_off, int cq_rank, const void* cq_norm, void* cq_out, int T);
 
 // Per-head products: out[t, h * out_head_stride + n] = sum_k a[t, h * a_head_stride + k] * w[h][n][k]
 // (w [heads, N, K]; rows of a and out are a_stride and out_stride apart; all three of `dtype`), times
@@ -324,6 +333,21 @@ int sp_delta(void* stream, int dtype, const void* mixed, long long mixed_stride,
 // max_q_len, scratch: as for sp_retention, with sp_delta_scratch_floats numbers.
 long long sp_delta_scratch_floats(int heads, int dim, int vdim, int n_seqs, int max_q_len, int T);
 
+// A matrix memory with exponential gates (mLSTM).  proj [T, stride] holds q and k (heads * dim each), v and an output gate
+// (heads * vdim each) and two numbers per head (i, f) at their offsets.  Per head: i = cap tanh((i + bias_i) / cap), f =
+// logsigmoid(cap tanh((f + bias_f) / cap)); with a running maximum m, which starts at 0: m' = max(f + m, i), S <- exp(f + m - m') S
+// + exp(i - m') v k^T, n <- exp(f + m - m') n + exp(i - m') k, and with q' = dim^(-1/2) q: o = S q' / (max(|n . q'|, exp(-m')) + 1e-6).
+// out [T, heads * vdim] = o / sqrt(mean over vdim of o^2 + eps) * norm[heads * vdim] * sigmoid(gate).  memory float32
+// [slots, heads, vdim + 1, dim]: S a row per value number, n as the last row; maxima float32 [slots, heads].  norm, biases
+// float32.
+int sp_mlstm_takes(int dim, int vdim);
+int sp_mlstm(void* stream, int dtype, const void* proj, long long stride, int q_off, int k_off, int v_off, int gate_off, int i_off,
+             int f_off, int heads, int dim, int vdim, float cap, const float* bias_i, const float* bias_f, const float* norm,
+             float eps, const int32_t* q_start, const int32_t* q_len, const int32_t* state_slots, float* memory, float* maxima,
+             void* out, int T, int n_seqs, int max_q_len, float* scratch);
+// max_q_len, scratch: as for sp_retention, with sp_mlstm_scratch_floats numbers.
+long long sp_mlstm_scratch_floats(int dtype, int heads, int dim, int vdim, int n_seqs, int max_q_len, int T);
+
 // ---- short causal convolutions, state-space scans and what goes with them (ssm.hip) ----
 // y[t, c] = act(bias[c] + sum_j w[c, j] x[t - taps + 1 + j, c]) (+ x[t, c] with add_input), a causal convolution over
 // time per channel within each request; inputs before a request's share of the step come from its state rows
@@ -338,7 +362,7 @@ int sp_short_conv(void* stream, int dtype, const void* x, long long x_stride, in
 // out [T, parts * size] = x / sqrt(mean over each part of x^2 + eps) * w, every row in `parts` equal parts, x float32.
 int sp_group_rmsnorm(void* stream, const float* x, int w_dtype, const void* w, float eps, int out_dtype, void* out, int T,
                      int parts, int size);
-// In place on n numbers of `dtype`: kind 0 = x * Phi(x), the exact (erf) GELU.
+// In place on n numbers of `dtype`: kind 0 = x * Phi(x), the exact (erf) GELU; 1 = max(x, 0)^2.
 int sp_activation(void* stream, int dtype, void* x, long long n, int kind);
 // out[p, :] = x[p / top, :] * weights[p]   (p < T * top; x, out of `dtype` [.., H]; weights float32)
 int sp_scale_rows(void* stream, int dtype, const void* x, const float* weights, int top, void* out, int T, int H);

@@ -175,6 +175,14 @@ __global__ __launch_bounds__(256) void gelu_erf_kernel(T* __restrict__ x, long l
 }
 
 template <typename T>
+__global__ __launch_bounds__(256) void relu_squared_kernel(T* __restrict__ x, long long n) {
+  for (long long i = blockIdx.x * 256ll + threadIdx.x; i < n; i += 256ll * gridDim.x) {
+    const float v = fmaxf(to_float(x[i]), 0.f);
+    x[i] = from_float<T>(v * v);
+  }
+}
+
+template <typename T>
 __global__ __launch_bounds__(256) void scale_rows_kernel(const T* __restrict__ x, const float* __restrict__ weights, int top,
                                                          T* __restrict__ out, int H) {
   const size_t p = blockIdx.x;
@@ -897,11 +905,14 @@ extern "C" int sp_group_rmsnorm(void* stream, const float* x, int w_dtype, const
 }
 
 extern "C" int sp_activation(void* stream, int dtype, void* x, long long n, int kind) {
-  SP_REQUIRE(kind == 0, "sp_activation: no activation %d (0 = the exact GELU)", kind);
+  SP_REQUIRE(kind == 0 || kind == 1, "sp_activation: no activation %d (0 = the exact GELU, 1 = the square of ReLU)", kind);
   SP_REQUIRE((dtype == kF32 || dtype == kBF16) && n >= 0 && (x || n == 0), "sp_activation: bad arguments");
   if (n == 0) return 0;
   const unsigned blocks = unsigned(n / 256 + 1 < 65536 ? n / 256 + 1 : 65536);
-  if (dtype == kF32) gelu_erf_kernel<float><<<blocks, 256, 0, (hipStream_t)stream>>>((float*)x, n);
+  if (kind == 1) {
+    if (dtype == kF32) relu_squared_kernel<float><<<blocks, 256, 0, (hipStream_t)stream>>>((float*)x, n);
+    else relu_squared_kernel<bf16_t><<<blocks, 256, 0, (hipStream_t)stream>>>((bf16_t*)x, n);
+  } else if (dtype == kF32) gelu_erf_kernel<float><<<blocks, 256, 0, (hipStream_t)stream>>>((float*)x, n);
   else gelu_erf_kernel<bf16_t><<<blocks, 256, 0, (hipStream_t)stream>>>((bf16_t*)x, n);
   return check_launch("sp_activation");
 }

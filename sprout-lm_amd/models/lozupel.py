@@ -9,8 +9,7 @@ from __future__ import annotations
 
 from ..config.base import ConfigError
 from ..config.lozupel import AttentionSizes, DeltaSizes, LozupelConfig
-from ..parts.base import make_part
-from .plan import LayerCall, LayerPlan, ModelParts, ModelPlan, PartPlan
+from .plan import LayerPlan, ModelPlan, PartPlan, run_schedule
 
 # The design gives no position limit; the engine's bookkeeping wants one.
 MAX_POSITIONS = 1 << 22
@@ -77,20 +76,6 @@ def _run_order(cfg: LozupelConfig) -> list[int]:
     return order + list(range(loop.stop, n))
 
 
-def _schedule(layers: list, order: list[int]) -> list:
-    """Every run of a layer keeps its pages, states and convolution inputs in cache slots of its own, numbered in the order
-    in which the runs' parts name them; what a part keeps is asked of the part itself."""
-    needs = []
-    for layer in layers:
-        block = make_part("block", layer.block, **{name: part.make() for name, part in layer.parts.items()})
-        needs.append(list(ModelParts.cache_needs(block)))
-    schedule, free = [], 0
-    for i in order:
-        schedule.append(LayerCall(i, {key: free + n for n, key in enumerate(needs[i])} or None))
-        free += len(needs[i])
-    return schedule
-
-
 def build_lozupel(cfg: LozupelConfig) -> ModelPlan:
     layers = [_layer(cfg, i) for i in range(len(cfg.layers))]
     if cfg.loop is not None:
@@ -99,6 +84,6 @@ def build_lozupel(cfg: LozupelConfig) -> ModelPlan:
         architecture=cfg.architecture, config=cfg, hidden_size=cfg.width, vocab_size=cfg.vocab, max_positions=MAX_POSITIONS,
         eos_token_ids=(), embedding=PartPlan("embedding", "token_embedding", {"vocab": cfg.vocab, "hidden": cfg.width,
                                                                               "tensor": "embed", "scale": cfg.embedding_scale}),
-        layers=layers, schedule=_schedule(layers, _run_order(cfg)), final_norm=_norm(cfg, "final.norm"),
+        layers=layers, schedule=run_schedule(layers, _run_order(cfg)), final_norm=_norm(cfg, "final.norm"),
         head=PartPlan("head", "linear_head", {"vocab": cfg.vocab, "hidden": cfg.width, "tied": False, "tensor": "head",
                                               "softcap": cfg.logit_softcap}))

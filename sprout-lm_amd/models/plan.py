@@ -217,3 +217,18 @@ class ModelParts:
             part.prepare(device, dtype)
         if getattr(self.head, "tied", False):
             self.head.tie(self.embedding.w["weight"])
+
+
+def run_schedule(layers: list[LayerPlan], order) -> list[LayerCall]:
+    """The run order `order` (layer numbers, a layer as often as it runs) in which every run of a layer keeps its pages,
+    states and convolution inputs in cache slots of its own, numbered in the order in which the runs' parts name them; what a
+    part keeps is asked of the part itself."""
+    needs = []
+    for layer in layers:
+        block = make_part("block", layer.block, **{name: part.make() for name, part in layer.parts.items()})
+        needs.append(list(ModelParts.cache_needs(block)))
+    schedule, free = [], 0
+    for i in order:
+        schedule.append(LayerCall(i, {key: free + n for n, key in enumerate(needs[i])} or None))
+        free += len(needs[i])
+    return schedule

@@ -254,29 +254,68 @@ def embed_bigram(table: torch.Tensor, pairs: torch.Tensor, tokens, positions, q_
                                     residual.data_ptr(), T, H, V, int(buckets), int(mul_prev), int(mul_cur)))
 
 
-def latent_prepare(proj: torch.Tensor, q_off: int, heads: int, dim: int, rot: int, dkv_off: int, rank: int,
-                   norm_weight: torch.Tensor, eps: float, positions, freq: torch.Tensor, rot_dims: int, magnitude: float,
-                   slot_mapping, k_pool, v_pool, q_out: torch.Tensor) -> None:
-    """From a row of projections: the normed latent and the turned shared key part into the pools (keys
-    [pages, 1, page, rank + rot], values [pages, 1, rank + rot, page], whose last rot columns are left alone), and
-    every head's turned query part into q_out[t, head, rank:] (see sprout_hip.h).  Float32 rows turn by float64 angles."""
-    _gpu(proj, "projections"); _gpu(norm_weight, "latent norm weight"); _gpu(q_out, "latent queries"); _gpu(freq, "frequencies")
-    T, stride = proj.shape
-    width = rank + rot
-    if tuple(q_out.shape) != (T, heads * width) or q_out.dtype != proj.dtype:
-        raise KernelError(f"latent_prepare: queries must be [{T}, {heads * width}] {proj.dtype}, got {tuple(q_out.shape)} {q_out.dtype}")
-    if norm_weight.numel() != rank or freq.dtype != torch.float64 or freq.numel() < rot_dims // 2:
-        raise KernelError("latent_prepare: the norm weight must hold rank numbers and freq rot_dims / 2 float64 numbers")
+LATENT_PAIRINGS = {"interleaved": 0, "halves": 1}      # which numbers of a latent's turned part turn together
+
+
+def latent_prepare(heads: int, dim: int, rot: int, rank: int, width: int, eps: float, positions, freq: torch.Tensor,
+                   rot_dims: int, magnitude: float, pairing: str, latent=None, queries=None, query_latent=None) -> None:
+    """What stands between the projections of latent attention and the attention kernel, each of three jobs where it is
+    asked for (see sprout_hip.h); float32 rows turn by float64 angles.
+
+    `latent` (rows, column, norm weight, slot_mapping, k_pool, v_pool): the normed latent and the turned shared key part
+    into the pools (keys [pages, 1, page, width], values [pages, 1, width, page] whose columns behind the latent are left
+    alone).  `queries` (rows, column, out): every head's turned part, column + h * (dim + rot) + dim on, to
+    out[t, h * width + rank:], zeros behind it.  `query_latent` (rows, column, norm weight, out): out = the RMS-normed
+    columns of the query latent."""
+    jobs = [job for job in (latent, queries, query_latent) if job is not None]
+    if not jobs:
+        return
+    T, dtype = jobs[0][0].shape[0], jobs[0][0].dtype
+    for job in jobs:
+        _gpu(job[0], "projections")
+        if job[0].shape[0] != T or job[0].dtype != dtype:
+            raise KernelError("latent_prepare: the rows of one call are of one dtype and as many tokens")
+    _gpu(freq, "frequencies")
+    if freq.dtype != torch.float64 or freq.numel() < rot_dims // 2 or width < rank + rot:
+        raise KernelError("latent_prepare: freq must hold rot_dims / 2 float64 numbers and the width a latent and its turned part")
     _ints(positions, T, "positions")
+    norm_code = None
     page_size = num_pages = 0
-    if slot_mapping is not None:
+
+    def norm_of(weight, size: int) -> None:
+        nonlocal norm_code
+        _gpu(weight, "latent norm weight")
+        code = _code(weight, "latent norm weight")
+        if weight.numel() != size or (norm_code is not None and norm_code != code):
+            raise KernelError(f"latent_prepare: norm weights must be of one dtype and hold {size} numbers here")
+        norm_code = code
+
+    kv = (None, 0, 0, None, None, None, None)
+    if latent is not None:
+        rows, column, weight, slot_mapping, k_pool, v_pool = latent
+        norm_of(weight, rank)
         _ints(slot_mapping, T, "slot_mapping")
-        num_pages, page_size = _check_pools(k_pool, v_pool, 1, width, proj.dtype, "latent_prepare")
-    check(library().sp_latent_prepare(_stream(), _code(proj, "projections"), proj.data_ptr(), stride, q_off, heads, dim, rot,
-                                      dkv_off, rank, _code(norm_weight, "latent norm weight"), norm_weight.data_ptr(),
-                                      float(eps), positions.data_ptr(), freq.data_ptr(), rot_dims, float(magnitude),
-                                      int(proj.dtype == torch.float32), _ptr(slot_mapping), _ptr(k_pool), _ptr(v_pool),
-                                      page_size, num_pages, q_out.data_ptr(), T))
+        num_pages, page_size = _check_pools(k_pool, v_pool, 1, width, dtype, "latent_prepare")
+        kv = (rows.data_ptr(), rows.shape[1], column, weight.data_ptr(), slot_mapping.data_ptr(), k_pool.data_ptr(), v_pool.data_ptr())
+    q = (None, 0, 0, None)
+    if queries is not None:
+        rows, column, out = queries
+        _gpu(out, "latent queries")
+        if tuple(out.shape) != (T, heads * width) or out.dtype != dtype:
+            raise KernelError(f"latent_prepare: queries must be [{T}, {heads * width}] {dtype}, got {tuple(out.shape)} {out.dtype}")
+        q = (rows.data_ptr(), rows.shape[1], column, out.data_ptr())
+    cq = (None, 0, 0, 0, None, None)
+    if query_latent is not None:
+        rows, column, weight, out = query_latent
+        _gpu(out, "query latents")
+        norm_of(weight, out.shape[1])
+        if out.shape[0] != T or out.dtype != dtype or not out.is_contiguous():
+            raise KernelError(f"latent_prepare: query latents must be [{T}, rank] {dtype}, got {tuple(out.shape)} {out.dtype}")
+        cq = (rows.data_ptr(), rows.shape[1], column, out.shape[1], weight.data_ptr(), out.data_ptr())
+    check(library().sp_latent_prepare(_stream(), _CODES[dtype], heads, dim, rot, rank, width, norm_code or 0, float(eps),
+                                      positions.data_ptr(), freq.data_ptr(), rot_dims, float(magnitude),
+                                      variant_code(LATENT_PAIRINGS, pairing, "rotation pairing"), int(dtype == torch.float32),
+                                      *kv, page_size, num_pages, *q, *cq, T))
 
 
 def head_gemm(a: torch.Tensor, a_offset: int, a_head_stride: int, w: torch.Tensor, out: torch.Tensor, out_offset: int,
@@ -450,22 +489,26 @@ def route_combine_identity(y: torch.Tensor, row_of_pair, ids: torch.Tensor, weig
 def qkv_prepare(proj: torch.Tensor, nq: int, nkv: int, dim: int, vdim: int, width: int, q_out: torch.Tensor, positions=None,
                 inv_freq=None, inv_freq_tail=None, rotary_dim: int = 0, q_norm=None, k_norm=None, eps: float = 0.0,
                 blend=None, first=None, keep_first: bool = False, slot_mapping=None, k_pool=None, v_pool=None,
-                magnitude: float = 1.0, head_norm: bool = False, q_mult: torch.Tensor | None = None, offset: int = 0) -> None:
+                magnitude: float = 1.0, head_norm: bool = False, q_mult: torch.Tensor | None = None, offset: int = 0,
+                maps: int = 1) -> None:
     """From rows of projections, from column `offset` on [q | k | v] (heads of `dim`, `dim` and `vdim` numbers): optional RMS norm over the whole
     q row and the whole k row, optional rotation of the heads' first rotary_dim numbers, optional blend of the values
     with `first` (or `first` <- values), q to q_out [T, nq * width], k and v into pools that keep both `width` wide
     (zeros behind); cosines and sines times `magnitude`; with `head_norm` every q and k head is divided, after turning,
     by its root mean square over dim (`eps` inside the root); `q_mult` (float32, one number per query head) multiplies the
-    turned queries; see sprout_hip.h."""
+    turned queries; `maps`: keys of `dim` numbers that a key head holds side by side, query row n being map n % maps of its
+    head (nq counts rows, nkv key/value heads); see sprout_hip.h."""
     _gpu(proj, "projections"); _gpu(q_out, "queries")
     T, stride = proj.shape
-    if offset < 0 or stride < offset + (nq + nkv) * dim + nkv * vdim or tuple(q_out.shape) != (T, nq * width) or q_out.dtype != proj.dtype:
+    if maps < 1 or nq % maps or width < maps * dim:
+        raise KernelError(f"qkv_prepare: {nq} query rows and a width of {width} do not hold {maps} maps of {dim} numbers a head")
+    if offset < 0 or stride < offset + (nq + nkv * maps) * dim + nkv * vdim or tuple(q_out.shape) != (T, nq * width) or q_out.dtype != proj.dtype:
         raise KernelError(f"qkv_prepare: rows of {stride} and queries {tuple(q_out.shape)} {q_out.dtype} do not fit the head sizes")
     if (q_norm is None) != (k_norm is None):
         raise KernelError("qkv_prepare: queries and keys are normed together or not at all")
     if q_norm is not None:
         _gpu(q_norm, "query norm"); _gpu(k_norm, "key norm")
-        if q_norm.dtype != proj.dtype or k_norm.dtype != proj.dtype or q_norm.numel() != nq * dim or k_norm.numel() != nkv * dim:
+        if q_norm.dtype != proj.dtype or k_norm.dtype != proj.dtype or q_norm.numel() != nq * dim or k_norm.numel() != nkv * maps * dim:
             raise KernelError("qkv_prepare: the norm weights must cover the whole q row and the whole k row")
     if rotary_dim:
         _ints(positions, T, "positions"); _gpu(inv_freq, "inv_freq")
@@ -493,7 +536,20 @@ def qkv_prepare(proj: torch.Tensor, nq: int, nkv: int, dim: int, vdim: int, widt
                                    int(rotary_dim), _ptr(blend), _ptr(first), int(bool(keep_first)), _ptr(slot_mapping),
                                    _ptr(k_pool) if slot_mapping is not None else None,
                                    _ptr(v_pool) if slot_mapping is not None else None, page_size, num_pages, q_out.data_ptr(), T,
-                                   float(magnitude), int(bool(head_norm)), _ptr(q_mult)))
+                                   float(magnitude), int(bool(head_norm)), _ptr(q_mult), int(maps)))
+
+
+def map_difference(maps: torch.Tensor, width: int, factor: torch.Tensor, eps: float, scale: float, out: torch.Tensor, heads: int,
+                   vdim: int) -> None:
+    """out[t, h] = rms(maps[t, 2 h] - factor * maps[t, 2 h + 1]) * scale over vdim of `width` numbers a map (`eps` inside the
+    root); `factor`: one float32 number on the device."""
+    _gpu(maps, "attention maps"); _gpu(out, "map difference"); _gpu(factor, "map factor")
+    T = out.shape[0]
+    if maps.shape[0] < T or maps.shape[1] != 2 * heads * width or tuple(out.shape) != (T, heads * vdim) or not out.is_contiguous() \
+            or not maps.is_contiguous() or factor.dtype != torch.float32 or factor.numel() != 1:
+        raise KernelError(f"map_difference: maps {tuple(maps.shape)}, factor and result {tuple(out.shape)} do not fit")
+    check(library().sp_map_difference(_stream(), _code(maps, "attention maps"), maps.data_ptr(), width, factor.data_ptr(),
+                                      float(eps), float(scale), _code(out, "map difference"), out.data_ptr(), T, heads, vdim))
 
 
 STORE, ACCUMULATE, STORE_F32 = 0, 1, 2
@@ -965,7 +1021,7 @@ def group_rmsnorm(x: torch.Tensor, weight: torch.Tensor, eps: float, out: torch.
                                      _code(out, "norm output"), out.data_ptr(), T, parts, n // parts))
 
 
-UNARY_ACTIVATIONS = {"gelu_erf": 0}      # x * Phi(x), the exact GELU
+UNARY_ACTIVATIONS = {"gelu_erf": 0, "relu_squared": 1}      # x * Phi(x), the exact GELU; max(x, 0)^2
 
 
 def activation(x: torch.Tensor, kind: str) -> None:
@@ -1124,6 +1180,40 @@ def retention(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, g_off: int
                                  heads, dim, vdim, rotary_dim, _ptr(cos_sin) if rotary_dim else None, decay.data_ptr(), float(eps),
                                  q_start.data_ptr(), q_len.data_ptr(), state_slots.data_ptr(), state.data_ptr(), out.data_ptr(),
                                  T, n_seqs, int(max_q_len) if scratch is not None else 0, _ptr(scratch)))
+
+
+def mlstm_takes(dim: int, vdim: int) -> bool:
+    return bool(library().sp_mlstm_takes(int(dim), int(vdim)))
+
+
+def mlstm(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, gate_off: int, i_off: int, f_off: int, heads: int, dim: int,
+          vdim: int, cap: float, bias_i: torch.Tensor, bias_f: torch.Tensor, norm: torch.Tensor, eps: float, q_start, q_len,
+          state_slots, n_seqs: int, memory: torch.Tensor, maxima: torch.Tensor, out: torch.Tensor, max_q_len: int = 0,
+          workspace=None) -> None:
+    """The matrix memory of sp_mlstm (sprout_hip.h) on a step's tokens.  `max_q_len`, `workspace`: as for `rglru`."""
+    T = out.shape[0]
+    _gpu(proj, "projections"); _gpu(out, "memory output"); _gpu(memory, "memory"); _gpu(maxima, "running maxima")
+    if proj.shape[0] < T or out.dtype != proj.dtype or tuple(out.shape) != (T, heads * vdim) or not out.is_contiguous():
+        raise KernelError(f"mlstm: projections {tuple(proj.shape)} {proj.dtype} and output {tuple(out.shape)} {out.dtype} do not fit")
+    if max(q_off, k_off) + heads * dim > proj.shape[1] or max(v_off, gate_off) + heads * vdim > proj.shape[1] \
+            or max(i_off, f_off) + heads > proj.shape[1] or min(q_off, k_off, v_off, gate_off, i_off, f_off) < 0:
+        raise KernelError("mlstm: a row of projections does not hold q, k, v and the gates")
+    for t, n, what in ((bias_i, heads, "input gate bias"), (bias_f, heads, "forget gate bias"), (norm, heads * vdim, "norm weight")):
+        _gpu(t, what)
+        if t.dtype != torch.float32 or t.numel() != n:
+            raise KernelError(f"mlstm: the {what} must hold {n} float32 values")
+    if memory.dtype != torch.float32 or tuple(memory.shape[1:]) != (heads, vdim + 1, dim) or not memory.is_contiguous() \
+            or maxima.dtype != torch.float32 or tuple(maxima.shape) != (memory.shape[0], heads) or not maxima.is_contiguous():
+        raise KernelError(f"mlstm: the memory must be float32 [slots, {heads}, {vdim + 1}, {dim}] beside [slots, {heads}] maxima")
+    for t, what in ((q_start, "q_start"), (q_len, "q_len"), (state_slots, "state_slots")):
+        _ints(t, n_seqs, what)
+    code = _code(proj, "projections")
+    need = library().sp_mlstm_scratch_floats(code, heads, dim, vdim, n_seqs, int(max_q_len), T) if workspace is not None else 0
+    scratch = _scan_scratch(need, workspace)
+    check(library().sp_mlstm(_stream(), code, proj.data_ptr(), proj.shape[1], q_off, k_off, v_off, gate_off, i_off, f_off, heads,
+                             dim, vdim, float(cap), bias_i.data_ptr(), bias_f.data_ptr(), norm.data_ptr(), float(eps),
+                             q_start.data_ptr(), q_len.data_ptr(), state_slots.data_ptr(), memory.data_ptr(), maxima.data_ptr(),
+                             out.data_ptr(), T, n_seqs, int(max_q_len) if scratch is not None else 0, _ptr(scratch)))
 
 
 def gemm_from_residual(residual: torch.Tensor, norm_weight: torch.Tensor, eps: float, w: torch.Tensor, out: torch.Tensor,

@@ -67,8 +67,9 @@ def _declare(lib):
         "sp_layernorm": [c_void, c_void, c_void, c_int, c_void, c_void, c_void, c_void, c_float, c_int, c_void, c_void, c_int, c_int],
         "sp_embed_bigram": [c_void, c_int, c_void, c_void, c_void, c_void, c_void, c_void, c_void, c_void, c_void, c_void,
                             c_int, c_int, c_int, c_i64, c_i64, c_i64],
-        "sp_latent_prepare": [c_void, c_int, c_void, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void, c_float,
-                              c_void, c_void, c_int, c_float, c_int, c_void, c_void, c_void, c_int, c_int, c_void, c_int],
+        "sp_latent_prepare": [c_void, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_void, c_void, c_int, c_float,
+                              c_int, c_int, c_void, c_int, c_int, c_void, c_void, c_void, c_void, c_int, c_int, c_void, c_int,
+                              c_int, c_void, c_void, c_int, c_int, c_int, c_void, c_void, c_int],
         "sp_head_gemm": [c_void, c_int, c_void, c_i64, c_i64, c_void, c_void, c_i64, c_i64, c_void, c_i64, c_int, c_int,
                          c_int, c_int],
         "sp_group_tile_rows": [c_int, c_i64, c_int, c_int],
@@ -83,7 +84,11 @@ def _declare(lib):
         "sp_route_combine_identity": [c_void, c_void, c_void, c_void, c_int, c_void, c_int, c_void, c_int, c_void, c_int, c_int],
         "sp_qkv_prepare": [c_void, c_int, c_void, c_i64, c_int, c_int, c_int, c_int, c_int, c_void, c_void, c_float, c_void,
                            c_void, c_void, c_int, c_void, c_void, c_int, c_void, c_void, c_void, c_int, c_int, c_void, c_int,
-                           c_float, c_int, c_void],
+                           c_float, c_int, c_void, c_int],
+        "sp_map_difference": [c_void, c_int, c_void, c_int, c_void, c_float, c_float, c_int, c_void, c_int, c_int, c_int],
+        "sp_mlstm_takes": [c_int] * 2,
+        "sp_mlstm": [c_void, c_int, c_void, c_i64, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_void,
+                     c_void, c_void, c_float, c_void, c_void, c_void, c_void, c_void, c_void, c_int, c_int, c_int, c_void],
         "sp_expert_down": [c_void, c_int, c_void, c_void, c_void, c_void, c_int, c_int, c_void, c_int, c_int, c_int, c_int],
         "sp_route_combine": [c_void, c_void, c_void, c_void, c_int, c_void, c_int, c_int],
         "sp_route_sigmoid": [c_void, c_void, c_void, c_void, c_int, c_int, c_int, c_int, c_void, c_void, c_void, c_void],
@@ -110,6 +115,8 @@ def _declare(lib):
     lib.sp_retention_scratch_floats.restype = c_i64
     lib.sp_delta_scratch_floats.argtypes = [c_int] * 6
     lib.sp_delta_scratch_floats.restype = c_i64
+    lib.sp_mlstm_scratch_floats.argtypes = [c_int] * 7
+    lib.sp_mlstm_scratch_floats.restype = c_i64
     lib.sp_ssd_scan_scratch_floats.argtypes = [c_int] * 5
     lib.sp_ssd_scan_scratch_floats.restype = c_i64
     lib.sp_selective_scan_scratch_floats.argtypes = [c_int] * 4

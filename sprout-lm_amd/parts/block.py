@@ -47,7 +47,8 @@ class PreNormBlock(Block):
 @register_part("block", "parallel")
 class ParallelBlock(Block):
     """x += mixer(norm_a(x)) + feed_forward(norm_b(x)): both norms read the same x, so both are taken before
-    either part adds into the float32 residual stream.  `ffn` (and its norm) may be absent."""
+    either part adds into the float32 residual stream.  `ffn` (and its norm) may be absent.  A feed-forward without a
+    norm of its own (`ffn_norm` None) reads norm_a(x), the mixer's input."""
 
     graph_safe = True
 
@@ -58,14 +59,16 @@ class ParallelBlock(Block):
 
     def parts(self):
         named = {"mixer_norm": self.mixer_norm, "mixer": self.mixer}
+        if self.ffn_norm is not None:
+            named["ffn_norm"] = self.ffn_norm
         if self.ffn is not None:
-            named.update({"ffn_norm": self.ffn_norm, "ffn": self.ffn})
+            named["ffn"] = self.ffn
         return named
 
     def forward(self, ctx, residual, caches):
         T, H = residual.shape
-        h = ctx.buffer("normed", (T, H), ctx.act_dtype)
-        if self.ffn is None:
+        h = h2 = ctx.buffer("normed", (T, H), ctx.act_dtype)
+        if self.ffn is None or self.ffn_norm is None:
             self.mixer_norm.forward(ctx, residual, h)
         else:
             h2 = ctx.buffer("normed_ffn", (T, H), ctx.act_dtype)

@@ -8,6 +8,7 @@ from ..cache.spec import PagedKVSpec
 from ..config.base import ConfigError
 from ..weights.loader import TensorSpec
 from .base import Mixer, register_part
+from .sink_attention import padded_width
 
 
 @register_part("mixer", "latent_attention")
@@ -15,6 +16,8 @@ class LatentAttention(Mixer):
     """Head h scores key j as (q_h[:dim] . (U_k,h c_j) + turn(q_h[dim:]) . turn(r_j)) * scale and sums values
     U_v,h c_j, where c_j (kv_rank numbers, RMS-normed) and r_j (rot_dim numbers) come from one down projection of
     token j; the head's output is multiplied by sigmoid(gate_h) where `gated`, and W_o mixes the heads.
+    q_rank: the queries come through a latent of their own, q = W_uq norm(W_dq h) (None: q = W_q h).  sinks: the softmax's
+    denominator also holds exp(sink_h), a tensor of one number per head that has no key and no value.
 
     Only c and turn(r) are cached, and attention runs on them directly: since q . (U_k c) = (U_k^T q) . c, the
     queries are carried into the latent's space by a per-head product, the attention kernels see ONE key/value
@@ -24,9 +27,12 @@ class LatentAttention(Mixer):
 
     hidden, heads, dim, rot_dim, vdim, kv_rank: sizes.  scale: the factor on q . k, used as given.  window: None,
     or how many of the latest keys (itself included) a query sees.  position: a PositionEncoding whose `freq`
-    (float64 table), `rotary_dim` (how many of the rot_dim numbers turn) and `magnitude` the turning kernel takes;
-    neighbours (2i, 2i + 1) turn together.  eps: of the latent's RMS norm.  `tensors`: local names of the query,
-    down, latent-norm, key-up, value-up, gate and output tensors.
+    (float64 table), `rotary_dim` (how many of the rot_dim numbers turn), `pairing` and `magnitude` the turning kernel
+    takes.  eps: of the latents' RMS norms.  `tensors`: local names of the query,
+    down, latent-norm, key-up, value-up, gate and output tensors; then of the query latent's down, norm and up tensors and
+    of the sinks.
+
+    Keys lie in the cache at `width` numbers, zeros behind (`padded_width`: a size the matrix-core kernels take).
     """
 
     graph_safe = True
@@ -35,64 +41,80 @@ class LatentAttention(Mixer):
 
     def __init__(self, hidden: int, heads: int, dim: int, rot_dim: int, vdim: int, kv_rank: int, scale: float, eps: float,
                  position, window: int | None = None, gated: bool = True, page_tokens: int | None = None,
-                 tensors: tuple = ("q", "dkv", "dkv.norm", "uk", "uv", "g", "o")):
+                 q_rank: int | None = None, sinks: bool = False, tensors: tuple = ()):
         if min(hidden, heads, dim, vdim, kv_rank) <= 0 or rot_dim < 0:
             raise ConfigError(f"Latent attention needs positive sizes, got heads={heads} dim={dim} rot_dim={rot_dim} "
                               f"vdim={vdim} kv_rank={kv_rank}.")
-        if getattr(position, "pairing", None) != "interleaved" and getattr(position, "rotary_dim", 0):
-            raise ConfigError("Latent attention turns neighbouring numbers; its position encoding must pair them so.")
+        if q_rank is not None and q_rank <= 0:
+            raise ConfigError(f"A query latent has a positive size, got {q_rank!r}.")
+        if getattr(position, "rotary_dim", 0) and getattr(position, "pairing", None) not in ops.LATENT_PAIRINGS:
+            raise ConfigError(f"Latent attention turns numbers in pairs {sorted(ops.LATENT_PAIRINGS)}; its position encoding must "
+                              f"pair them so.")
         if getattr(position, "rotary_dim", 0) > rot_dim:
             raise ConfigError(f"{position.rotary_dim} numbers cannot turn in a rotated part of {rot_dim}.")
-        try:      # one key/value head of width kv_rank + rot_dim under all query heads
-            ops.check_attention_sizes(heads, 1, kv_rank + rot_dim)
+        self.key_width = kv_rank + rot_dim
+        self.width = padded_width(self.key_width, self.key_width)
+        try:      # one key/value head of this width under all query heads
+            ops.check_attention_sizes(heads, 1, self.width)
         except ops.KernelError as error:
             raise ConfigError(str(error)) from None
         self.hidden, self.heads, self.dim, self.rot_dim, self.vdim, self.kv_rank = hidden, heads, dim, rot_dim, vdim, kv_rank
         self.scale, self.eps, self.position, self.window, self.gated = float(scale), float(eps), position, window, gated
-        self.page_tokens = page_tokens
-        self.names = tuple(tensors)
-        self.key_width = kv_rank + rot_dim
+        self.page_tokens, self.q_rank, self.sinks = page_tokens, q_rank, bool(sinks)
+        defaults = ("q", "dkv", "dkv.norm", "uk", "uv", "g", "o", "dq", "dq.norm", "uq", "sink")
+        self.names = tuple(tensors) + defaults[len(tensors):]
 
     # ------------------------------------------------------------------ what it keeps and costs
     def cache_spec(self):
-        return PagedKVSpec(1, self.key_width, self.window, self.page_tokens)
+        return PagedKVSpec(1, self.width, self.window, self.page_tokens)
 
     def cache_elements_per_token(self) -> int:
-        return 2 * self.key_width
+        return 2 * self.width
 
     def flops(self, tokens: int, pairs: int = 0) -> float:
         H = self.heads
-        rows_in = H * (self.dim + self.rot_dim) + self.key_width + (H if self.gated else 0)
-        products = rows_in * self.hidden + H * self.dim * self.kv_rank + H * self.kv_rank * self.vdim + H * self.vdim * self.hidden
-        return 2.0 * tokens * products + 4.0 * H * self.key_width * pairs
+        query_rows = H * (self.dim + self.rot_dim)
+        rows_in = (self.q_rank or query_rows) + self.key_width + (H if self.gated else 0)
+        products = rows_in * self.hidden + (self.q_rank or 0) * query_rows + H * self.dim * self.kv_rank \
+            + H * self.kv_rank * self.vdim + H * self.vdim * self.hidden
+        return 2.0 * tokens * products + 2.0 * H * (self.key_width + self.kv_rank) * pairs
 
     def tensors(self):
-        q, dkv, norm, uk, uv, g, o = self.names
-        H = self.heads
-        out = {q: TensorSpec((H * (self.dim + self.rot_dim), self.hidden)),
-               dkv: TensorSpec((self.key_width, self.hidden)),
-               norm: TensorSpec((self.kv_rank,), "vector", "one_plus_normal"),
-               uk: TensorSpec((H * self.dim, self.kv_rank)),
-               uv: TensorSpec((H * self.vdim, self.kv_rank)),
-               o: TensorSpec((self.hidden, H * self.vdim))}
+        q, dkv, norm, uk, uv, g, o, dq, dq_norm, uq, sink = self.names
+        H, rows = self.heads, self.heads * (self.dim + self.rot_dim)
+        if self.q_rank is None:
+            out = {q: TensorSpec((rows, self.hidden))}
+        else:
+            out = {dq: TensorSpec((self.q_rank, self.hidden)), dq_norm: TensorSpec((self.q_rank,), "vector", "one_plus_normal"),
+                   uq: TensorSpec((rows, self.q_rank))}
+        out.update({dkv: TensorSpec((self.key_width, self.hidden)),
+                    norm: TensorSpec((self.kv_rank,), "vector", "one_plus_normal"),
+                    uk: TensorSpec((H * self.dim, self.kv_rank)),
+                    uv: TensorSpec((H * self.vdim, self.kv_rank)),
+                    o: TensorSpec((self.hidden, H * self.vdim))})
         if self.gated:
             out[g] = TensorSpec((H, self.hidden))
+        if self.sinks:
+            out[sink] = TensorSpec((H,), "vector")
         return out
 
     def bind(self, tensors):
-        q, dkv, norm, uk, uv, g, o = self.names
+        q, dkv, norm, uk, uv, g, o, dq, dq_norm, uq, sink = self.names
         H = self.heads
-        # one product for everything that reads the mixer's input: queries, latent + rotated key part, gates
-        # (rows of zeros behind them bring a row of results to a multiple of 8 numbers: every token's row, and with
+        # one product for everything that reads the mixer's input: queries (or their latent), latent + rotated key part,
+        # gates (rows of zeros behind them bring a row of results to a multiple of 8 numbers: every token's row, and with
         # head sizes in eights every head's part of it, then starts at a multiple of 16 bytes for the per-head products)
-        stacked = [tensors[q], tensors[dkv]] + ([tensors[g]] if self.gated else [])
+        first = tensors[q if self.q_rank is None else dq]
+        stacked = [first, tensors[dkv]] + ([tensors[g]] if self.gated else [])
         rows = sum(t.shape[0] for t in stacked)
         if rows % 8:
-            stacked.append(torch.zeros(8 - rows % 8, self.hidden, dtype=tensors[q].dtype, device=tensors[q].device))
+            stacked.append(torch.zeros(8 - rows % 8, self.hidden, dtype=first.dtype, device=first.device))
         self.w_in = torch.cat(stacked, dim=0).contiguous()
-        self.q_off, self.dkv_off = 0, H * (self.dim + self.rot_dim)
+        self.q_off, self.dkv_off = 0, first.shape[0]
         self.gate_off = self.dkv_off + self.key_width
         self.w_norm = tensors[norm]
+        self.w_q_norm, self.w_uq = (None, None) if self.q_rank is None else (tensors[dq_norm], tensors[uq])
+        self.sink = tensors[sink].to(torch.float32).contiguous() if self.sinks else None
         # U_k per head as [kv_rank, dim]: the product that carries a query into the latent's space
         self.w_uk_t = tensors[uk].view(H, self.dim, self.kv_rank).transpose(1, 2).contiguous()
         self.w_uv = tensors[uv].view(H, self.vdim, self.kv_rank).contiguous()
@@ -107,20 +129,29 @@ class LatentAttention(Mixer):
 
     # ------------------------------------------------------------------ the step
     def forward(self, ctx, h, residual, cache):
-        T, H, W = h.shape[0], self.heads, self.key_width
+        T, H, W = h.shape[0], self.heads, self.width
         proj = ctx.buffer("latent_proj", (T, self.w_in.shape[0]), ctx.act_dtype)
         ops.gemm(h, self.w_in, proj)
         queries = ctx.buffer("latent_q", (T, H * W), ctx.act_dtype)
         writes = cache.writes
-        ops.latent_prepare(proj, self.q_off, H, self.dim, self.rot_dim, self.dkv_off, self.kv_rank, self.w_norm, self.eps,
-                           ctx.positions, self.position.freq, self.position.rotary_dim, self.position.magnitude,
-                           cache.slot_mapping if writes else None, cache.k if writes else None,
-                           cache.v if writes else None, queries)
-        ops.head_gemm(proj, self.q_off, self.dim + self.rot_dim, self.w_uk_t, queries, 0, W)
+        turn = (ctx.positions, self.position.freq, self.position.rotary_dim, self.position.magnitude, self.position.pairing)
+        latent = (proj, self.dkv_off, self.w_norm, cache.slot_mapping, cache.k, cache.v) if writes else None
+        rows = proj
+        if self.q_rank is None:
+            ops.latent_prepare(H, self.dim, self.rot_dim, self.kv_rank, W, self.eps, *turn, latent=latent,
+                               queries=(proj, self.q_off, queries))
+        else:      # both latents in one launch, the queries' product, then their turn
+            c_q = ctx.buffer("latent_cq", (T, self.q_rank), ctx.act_dtype)
+            ops.latent_prepare(H, self.dim, self.rot_dim, self.kv_rank, W, self.eps, *turn, latent=latent,
+                               query_latent=(proj, self.q_off, self.w_q_norm, c_q))
+            rows = ctx.buffer("latent_uq", (T, self.w_uq.shape[0]), ctx.act_dtype)
+            ops.gemm(c_q, self.w_uq, rows)
+            ops.latent_prepare(H, self.dim, self.rot_dim, self.kv_rank, W, self.eps, *turn, queries=(rows, 0, queries))
+        ops.head_gemm(rows, self.q_off, self.dim + self.rot_dim, self.w_uk_t, queries, 0, W)
         mixed = ctx.buffer("latent_mixed", (T, H * W), ctx.act_dtype)
         ops.attention(queries, H * W, cache.k, cache.v, cache.block_tables, ctx.attention, mixed, H, 1, W, self.window,
                       self.scale, workspace=lambda n: ctx.buffer("attention_partials", (n,), torch.float32),
-                      kind=ctx.attention_kind)
+                      kind=ctx.attention_kind, sinks=self.sink)
         values = ctx.buffer("latent_values", (T, H * self.vdim), ctx.act_dtype)
         ops.head_gemm(mixed, 0, W, self.w_uv, values, 0, self.vdim, gate=proj if self.gated else None,
                       gate_offset=self.gate_off)

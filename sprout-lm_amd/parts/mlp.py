@@ -96,7 +96,7 @@ class GatedMLP(FeedForward):
 @register_part("feed_forward", "mlp")
 class DenseMLP(FeedForward):
     """down(act(up(x) + b_up)) + b_down, no gate.  `activation`: one of `ops.UNARY_ACTIVATIONS` ("gelu_erf": the exact
-    GELU, x * Phi(x)).  `bias`: the suffix of the biases' names, None for projections without them.  `tensors`: local
+    GELU, x * Phi(x); "relu_squared": max(x, 0)^2).  `bias`: the suffix of the biases' names, None for projections without them.  `tensors`: local
     names of the up and down matrices."""
 
     graph_safe = True

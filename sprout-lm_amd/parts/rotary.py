@@ -16,7 +16,13 @@ class NeoxRotary(PositionEncoding):
     min(ceil(turns(slow)), rotary_dim - 1) and ramp_d = clamp((d - lo) / max(hi - lo, 0.001), 0, 1) pair d turns by
     position * (f_d / factor * ramp_d + f_d * (1 - ramp_d)).
 
-    The table of inverse frequencies is computed in float64 and kept in float32; angles, sines
+    With the keys factor / original / low / high instead, frequencies are blended by wavelength ("Llama 3.1"), cosine and
+    sine as they are (`magnitude` 1): with turns = original f_d / (2 pi), the turns that the original context holds, pair d
+    keeps f_d where turns > high, takes f_d / factor where turns < low, and between them s f_d + (1 - s) f_d / factor with
+    s = (turns - low) / (high - low).
+
+    The table of inverse frequencies is computed in float64 and kept in float32 (`freq`: in float64 on the device, for the
+    kernels that turn a latent's part); angles, sines
     and cosines are float32 in the kernel.  For float32 models the part also keeps what the float32
     table lost (`inv_freq_tail`), and the kernel computes angle, sine and cosine in float64: a float32
     angle is off by up to position * 6e-8, more than every other rounding of that path together once
@@ -35,7 +41,9 @@ class NeoxRotary(PositionEncoding):
         if self.rotary_dim % 2 or not 0 < self.rotary_dim <= head_dim:
             raise ValueError(f"rotary_dim {self.rotary_dim} must be even and at most head_dim {head_dim}.")
         self.scaling = dict(scaling) if scaling else None
-        self.magnitude = 0.1 * math.log(float(self.scaling["factor"])) + 1.0 if self.scaling else 1.0
+        self.by_wavelength = bool(self.scaling) and "low" in self.scaling
+        self.magnitude = 0.1 * math.log(float(self.scaling["factor"])) + 1.0 if self.scaling and not self.by_wavelength else 1.0
+        self.freq = None
         self.inv_freq = None
         self.inv_freq_tail = None
 
@@ -48,6 +56,11 @@ class NeoxRotary(PositionEncoding):
         if not self.scaling:
             return freq
         factor, original = float(self.scaling["factor"]), float(self.scaling["original"])
+        if self.by_wavelength:
+            low, high = float(self.scaling["low"]), float(self.scaling["high"])
+            held = original * freq / (2.0 * math.pi)
+            share = ((held - low) / max(high - low, 1e-300)).clamp(0.0, 1.0)
+            return share * freq + (1.0 - share) * freq / factor
         turns = lambda t: n * math.log(original / (2.0 * math.pi * t)) / (2.0 * math.log(float(self.theta)))
         lo = max(math.floor(turns(float(self.scaling["fast"]))), 0)
         hi = min(math.ceil(turns(float(self.scaling["slow"]))), n - 1)
@@ -56,6 +69,7 @@ class NeoxRotary(PositionEncoding):
 
     def prepare(self, device, dtype):
         exact = self.frequencies()
+        self.freq = exact.to(device)
         self.inv_freq = exact.to(torch.float32).to(device)
         if dtype == torch.float32:
             self.inv_freq_tail = (exact - exact.to(torch.float32).to(torch.float64)).to(torch.float32).to(device)
@@ -133,9 +147,13 @@ class NoPosition(PositionEncoding):
 
     graph_safe_portions = True
 
+    magnitude = 1.0
+
     def __init__(self, head_dim: int = 0):
         self.head_dim = head_dim
+        self.freq = None
         self.inv_freq = None
 
     def prepare(self, device, dtype):
+        self.freq = torch.zeros(1, dtype=torch.float64, device=device)
         self.inv_freq = torch.zeros(1, dtype=torch.float32, device=device)

@@ -87,6 +87,9 @@ def _register_builtin():
     from .config.lozupel import LozupelConfig
     from .models.lozupel import build_lozupel
     register_architecture(LozupelConfig.architecture, LozupelConfig, build_lozupel)
+    from .config.varunex import VarunexConfig
+    from .models.varunex import build_varunex
+    register_architecture(VarunexConfig.architecture, VarunexConfig, build_varunex)
 
 
 _register_builtin()

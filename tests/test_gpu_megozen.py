@@ -185,9 +185,10 @@ def test_latent_norm_rotation_and_cache_write(dtype, heads, dim, rot, rot_dims, 
     k_pool = torch.full((pages, 1, page, width), 9.0, dtype=dtype, device=DEV)
     v_pool = torch.full((pages, 1, width, page), 9.0, dtype=dtype, device=DEV)
     q_out = torch.full((T, heads * width), 5.0, dtype=dtype, device=DEV)
-    ops.latent_prepare(dev(proj, dtype), q_off, heads, dim, rot, dkv_off, rank, dev(w_norm, dtype), eps,
-                       dev(positions, torch.int32), position.freq, rot_dims, position.magnitude,
-                       dev(slots, torch.int32), k_pool, v_pool, q_out)
+    rows = dev(proj, dtype)
+    ops.latent_prepare(heads, dim, rot, rank, width, eps, dev(positions, torch.int32), position.freq, rot_dims, position.magnitude,
+                       "interleaved", latent=(rows, dkv_off, dev(w_norm, dtype), dev(slots, torch.int32), k_pool, v_pool),
+                       queries=(rows, q_off, q_out))
     angle = np.float64 if dtype == torch.float32 else np.float32
     c = M.rms_norm(proj[:, dkv_off:dkv_off + rank], w_norm, eps)
     r = M.rotate_interleaved(proj[:, dkv_off + rank:dkv_off + width], positions, rot_cfg, angle) if rot else np.zeros((T, 0))
