@@ -36,6 +36,10 @@ def plain_side(folder: str, dtype: str):
         from tests.plain import lozupel_plain as Z
         cfg, weights = Z.load_folder(folder)
         return cfg, weights, Z.forward
+    if name == "Varunex":
+        from tests.plain import varunex_plain as V
+        cfg, weights = V.load_folder(folder)
+        return cfg, weights, V.forward
     if name == "Megozen":
         from tests.plain import megozen_plain as M
         cfg, weights = M.load_folder(folder)
