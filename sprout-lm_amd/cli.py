@@ -2,7 +2,7 @@
 
     python -m sprout_lm_amd demo [--json] [--pressure]
     python -m sprout_lm_amd generate MODEL_DIR --prompt-ids 1,2,3 [--max-new-tokens N] ...
-    python -m sprout_lm_amd init --preset tiny-a|tiny-b|qwen2.5-0.5b|megozen-s|bogilix-s|morarax-s|kodezen-s|lozupel-s|... | --config FILE  --out DIR [--seed N]
+    python -m sprout_lm_amd init --preset tiny-a|tiny-b|qwen2.5-0.5b|megozen-s|bogilix-s|morarax-s|kodezen-s|lozupel-s|varunex-s|... | --config FILE  --out DIR [--seed N]
 
 `demo` is the counterpart of the reference's src/demo.ts, with the reference's two options: a few requests on a
 tiny random model, told round by round (--json: the same as one JSON document; --pressure: a pool so small that
@@ -201,6 +201,37 @@ PRESETS.update({
     # large: 6 layers of width 4,096, two of them run twice (8 runs)
     "lozupel-l": _lozupel_preset(4096, 6, (2, 4, 2), 32, 4, 128, 32, 128, 8192, 32768),
     "lozupel-l-twin": _morarax_preset(4096, 8, 32, 4, 128, 32, 16, 8192, 32768),
+})
+
+
+def _varunex_preset(width: int, layers: int, heads: int, kv_heads: int, dim: int, latent: tuple, memory: tuple, ff: int, vocab: int) -> dict:
+    """A Varunex configuration: layers in the order latent attention, memory, differential attention, memory, again and again.
+    latent: heads, their unrotated and rotated numbers, the query and the key/value latents' sizes; memory: heads, key and value
+    numbers; differential attention: `heads` heads of two maps of `dim` numbers over values of 2 dim in a window of 1,024 keys.
+    Feed-forwards of ff * 3 / 2 inner numbers: two matrices where a gated one has three."""
+    lat_heads, lat_dim, rot_dim, q_rank, kv_rank = latent
+    attention = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": 2 * dim, "scale": dim ** -0.5, "diff": 0.5,
+                 "mask": {"size": 1024}, "rot": {"base": 500000.0, "dims": dim,
+                                                 "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}
+    latents = {"heads": lat_heads, "dim": lat_dim, "rot_dim": rot_dim, "vdim": lat_dim, "q_rank": q_rank, "kv_rank": kv_rank,
+               "scale": (lat_dim + rot_dim) ** -0.5, "rot": {"base": 10000.0, "dims": rot_dim}}
+    cells = {"heads": memory[0], "dim": memory[1], "vdim": memory[2], "gate_cap": 15.0}
+    order = (("latent_attention", latents), ("mlstm", cells), ("attention", attention), ("mlstm", cells))
+    entries = [{"type": order[i % 4][0], "mixer": order[i % 4][1], "mlp": {"kind": "dense", "ff": ff * 3 // 2}} for i in range(layers)]
+    return {"architecture": "Varunex", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "layers": entries}
+
+
+PRESETS.update({
+    # beside each the closest design the engine has at equal width, layers, attention heads and feed-forward work: Morarax
+    # small: keys of 96 + 32 beside each other, memories of 4 heads of 128 x 256
+    "varunex-s": _varunex_preset(1024, 8, 16, 2, 32, (16, 64, 32, 384, 96), (4, 128, 256), 2048, 32768),
+    "varunex-s-twin": _morarax_preset(1024, 8, 16, 2, 64, 8, 16, 2048, 32768),
+    # medium: latents of 128 + 64, memories of 8 heads of 128 x 256
+    "varunex-m": _varunex_preset(2048, 12, 16, 2, 64, (16, 128, 64, 768, 128), (8, 128, 256), 4224, 32768),
+    "varunex-m-twin": _morarax_preset(2048, 12, 16, 2, 128, 16, 16, 4224, 32768),
+    # large: latents of 192 + 64, memories of 8 heads of 256 x 512
+    "varunex-l": _varunex_preset(4096, 8, 32, 4, 64, (32, 128, 64, 1536, 192), (8, 256, 512), 8192, 32768),
+    "varunex-l-twin": _morarax_preset(4096, 8, 32, 4, 128, 32, 16, 8192, 32768),
 })
 
 

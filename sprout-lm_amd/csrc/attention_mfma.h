@@ -593,9 +593,49 @@ __global__ __launch_bounds__(64 * WPT * HPB) void attention_prefill_staged_kerne
     }
     __syncthreads();
   };
+  // A stage that takes more registers than a wave has to spare (wide heads on four waves) travels in pieces of eight: no
+  // register is held while the stage before is used.
+  constexpr bool PIECES = HD > 128 && !AHEAD;
+  auto bring = [&](int key0, auto in_lds) __attribute__((always_inline)) {
+    const bool interior = key0 >= f_lo && key0 + kStageKeys - 1 <= f_hi;
+    __syncthreads();
+#pragma unroll 1
+    for (int u0 = 0; u0 < PER_THREAD; u0 += 8) {
+      uint4 piece[8];
+#pragma unroll
+      for (int u = 0; u < 8; ++u) {
+        const int i = threadIdx.x + THREADS * (u0 + u);
+        if (i < KCHUNKS) {
+          const int r = i / (HD / 8), c = i % (HD / 8);
+          int key = key0 + r;
+          if (!interior) key = min(max(key, f_lo), f_hi);
+          piece[u] = ldg128(kbase + (((size_t(page_at(key, in_lds)) * heads) << page_shift) + (key & page_mask)) * HD + 8 * c);
+        } else if (i < CHUNKS) {
+          const int j = i - KCHUNKS, d = j / (kStageKeys / 8), c = j % (kStageKeys / 8);
+          int kb = key0 + 8 * c;
+          if (!interior) kb = min(max(kb, (f_lo >> 3) << 3), (f_hi >> 3) << 3);
+          piece[u] = ldg128(vbase + ((size_t(page_at(kb, in_lds)) * heads * HD + size_t(d)) << page_shift) + (kb & page_mask));
+        }
+      }
+#pragma unroll
+      for (int u = 0; u < 8; ++u) {
+        const int i = threadIdx.x + THREADS * (u0 + u);
+        if (i < KCHUNKS) {
+          const int r = i / (HD / 8), c = i % (HD / 8);
+          *reinterpret_cast<uint4*>(&ks[step_row(r) * KP + 8 * c]) = piece[u];
+        } else if (i < CHUNKS) {
+          const int j = i - KCHUNKS, d = j / (kStageKeys / 8), c = j % (kStageKeys / 8);
+          *reinterpret_cast<uint4*>(&vs[d * VP + 8 * c]) = piece[u];
+        }
+      }
+    }
+    __syncthreads();
+  };
   // this wave's keys of the stage that lies in LDS, 32 at a time
   auto use_stage = [&](int key0) __attribute__((always_inline)) {
-#pragma unroll
+    // (a wave that takes whole stages takes their steps one after the other: unrolled, their operands would not fit)
+    constexpr int UNROLL = WPT == 1 ? 1 : WAVE_KEYS / 32;
+#pragma unroll UNROLL
     for (int sub = 0; sub < WAVE_KEYS / 32; ++sub) {
       const int skey = WAVE_KEYS * wave + 32 * sub;
       const int wkey = key0 + skey;
@@ -622,7 +662,7 @@ __global__ __launch_bounds__(64 * WPT * HPB) void attention_prefill_staged_kerne
       }
     }
   };
-  uint4 stage[PER_THREAD];
+  uint4 stage[PIECES ? 1 : PER_THREAD];
   __syncthreads();   // the page numbers are in LDS
   if (st.keep > 0 && split == 0) {
     // the stages of kept first keys that lie wholly before the window's first stage: the block of the first split walks
@@ -631,19 +671,31 @@ __global__ __launch_bounds__(64 * WPT * HPB) void attention_prefill_staged_kerne
     f_lo = 0;
     f_hi = min(st.keep - 1, k_hi);
     for (int key0 = 0; key0 < min(st.keep, lo_stage); key0 += kStageKeys) {
-      fetch_from(stage, key0, std::false_type{});
-      to_lds(stage);
+      if constexpr (PIECES) {
+        bring(key0, std::false_type{});
+      } else {
+        fetch_from(stage, key0, std::false_type{});
+        to_lds(stage);
+      }
       use_stage(key0);
     }
     f_lo = window_lo;
     f_hi = k_hi;
   }
-  if (AHEAD && range_lo <= range_hi) fetch(stage, range_lo);
-  for (int key0 = range_lo; key0 <= range_hi; key0 += kStageKeys) {
-    if (!AHEAD) fetch(stage, key0);
-    to_lds(stage);
-    if (AHEAD && key0 + kStageKeys <= range_hi) fetch(stage, key0 + kStageKeys);
-    use_stage(key0);
+  if constexpr (PIECES) {
+    for (int key0 = range_lo; key0 <= range_hi; key0 += kStageKeys) {
+      if (table_in_lds) bring(key0, std::true_type{});
+      else bring(key0, std::false_type{});
+      use_stage(key0);
+    }
+  } else {
+    if (AHEAD && range_lo <= range_hi) fetch(stage, range_lo);
+    for (int key0 = range_lo; key0 <= range_hi; key0 += kStageKeys) {
+      if (!AHEAD) fetch(stage, key0);
+      to_lds(stage);
+      if (AHEAD && key0 + kStageKeys <= range_hi) fetch(stage, key0 + kStageKeys);
+      use_stage(key0);
+    }
   }
 
   // merge the waves of each team in turn: [wave][row][HD + 4] floats = (O^T row ..., maximum, sum, two unused).
@@ -1059,9 +1111,13 @@ static bool staged_prefill(int page_size) { return page_size >= 8 && (page_size 
 // four teams of four waves.  Above that the registers of 16 waves do not suffice: four teams of two waves
 // (each wave then takes 64 keys of a stage).  Three teams were slower than two or four at every size.
 // A portion of 2,048 tokens at a context of 32,768: 835 -> 472 us (14 heads of 64), 2,350 -> 1,470 us (28 of 128).
+// Head sizes above 128 (a latent beside its turned part): one wave a head, four heads a block, so that a stage, which takes
+// most of the LDS, still serves four heads; a group of fewer heads, or a head of 256 (whose sums alone take half of a wave's
+// registers): four waves a head, a head a block.
 struct StagedShape { int hpb, wpt; bool ahead; };
 static StagedShape staged_shape(int nq, int nkv, int hd, int n_tiles) {
   const int G = nq / nkv;
+  if (hd > 128) return G >= 3 && hd <= 192 ? StagedShape{4, 1, false} : StagedShape{1, 4, false};
   if (G <= 1) return {1, 4, false};
   if (G == 2) return {2, 4, hd > 64};
   if (hd > 64) return {4, 2, false};
@@ -1129,7 +1185,10 @@ static int launch_mfma(hipStream_t s, const void* q, int q_stride, const void* k
       qp, q_stride, kp, vp, block_tables, max_blocks, q_start, q_len, ctx_len, tiles, (uint16_t*)out, part_o,   \
       part_ml, splits, per_split, nq, nkv, page_shift, num_pages, st, scale2, n_tiles)
       // the same cases as staged_shape() and staged_paired()
-      if (paired) {
+      if constexpr (DT > 8) {
+        if (DT <= 12 && shape.hpb == 4) { if (paired) SP_STAGED(DT <= 12 ? 4 : 1, DT <= 12 ? 1 : 4, false, true); else SP_STAGED(DT <= 12 ? 4 : 1, DT <= 12 ? 1 : 4, false, false); }
+        else { if (paired) SP_STAGED(1, 4, false, true); else SP_STAGED(1, 4, false, false); }
+      } else if (paired) {
         if (shape.hpb == 1) SP_STAGED(1, 4, false, true);
         else if (shape.hpb == 2) SP_STAGED(2, 4, true, true);
         else { if constexpr (DT > 4) SP_STAGED(4, 2, false, true); else SP_STAGED(4, 4, true, true); }

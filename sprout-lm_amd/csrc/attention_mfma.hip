@@ -6,7 +6,7 @@ namespace sprout {
 
 bool attention_mfma_supports(int hd, int page_size, int nq, int nkv) {
   const int dt = hd / 16;
-  const bool hd_ok = hd % 16 == 0 && (dt <= 6 || dt == 8);
+  const bool hd_ok = hd % 16 == 0 && (dt <= 6 || dt == 8 || dt == 10 || dt == 12 || dt == 16);
   return hd_ok && page_size % 4 == 0;
 }
 bool attention_mfma_decode_supports(int nq, int nkv) { return true; }
@@ -32,6 +32,12 @@ size_t attention_decode_workspace_floats(int n_decode, int nq, int hd, int max_c
   return splits <= 1 ? 0 : size_t(n_decode) * nq * splits * (hd + 2);
 }
 
+int attention_mfma_wide(hipStream_t s, const void* q, int q_stride, const void* k_pool, const void* v_pool,
+                        const int32_t* block_tables, int max_blocks, const int32_t* q_start, const int32_t* q_len,
+                        const int32_t* ctx_len, const int32_t* tiles, int n_tiles, const int32_t* decode_seqs, int n_decode,
+                        int max_decode_ctx, int max_tile_ctx, int mean_tile_walk, float* workspace, void* out, int nq, int nkv,
+                        int hd, int page_size, int num_pages, ScoreStage st, float scale);
+
 int attention_mfma(hipStream_t s, const void* q, int q_stride, const void* k_pool, const void* v_pool,
                    const int32_t* block_tables, int max_blocks, const int32_t* q_start, const int32_t* q_len,
                    const int32_t* ctx_len, const int32_t* tiles, int n_tiles, const int32_t* decode_seqs, int n_decode,
@@ -44,6 +50,10 @@ int attention_mfma(hipStream_t s, const void* q, int q_stride, const void* k_poo
                            workspace, out, nq, nkv, page_size, num_pages, st, scale)
   switch (hd / 16) {
     SP_MFMA(1); SP_MFMA(2); SP_MFMA(3); SP_MFMA(4); SP_MFMA(5); SP_MFMA(6); SP_MFMA(8);
+    default:
+      return attention_mfma_wide(s, q, q_stride, k_pool, v_pool, block_tables, max_blocks, q_start, q_len, ctx_len, tiles, n_tiles,
+                                 decode_seqs, n_decode, max_decode_ctx, max_tile_ctx, mean_tile_walk, workspace, out, nq, nkv, hd,
+                                 page_size, num_pages, st, scale);
   }
 #undef SP_MFMA
   set_error("sp_attention: no matrix-core kernel for head size %d", hd);
@@ -56,7 +66,7 @@ int attention_mfma(hipStream_t s, const void* q, int q_stride, const void* k_poo
 // projection kernels of their own: 8 sequences 8,250 against 7,930, 24 sequences 21,870 against 21,260, 32
 // sequences 27,400 against 26,660, 64 sequences 39,840 against 40,350).
 bool attention_decode_project_takes(int hd, int page_size, int nq, int nkv, int n_decode, int max_decode_ctx, int hidden) {
-  if (!attention_mfma_supports(hd, page_size, nq, nkv) || !attention_mfma_decode_supports(nq, nkv)) return false;
+  if (hd > 128 || !attention_mfma_supports(hd, page_size, nq, nkv) || !attention_mfma_decode_supports(nq, nkv)) return false;
   const int n_splits = (max_decode_ctx + kDecodeChunk - 1) / kDecodeChunk;
   return n_decode >= 1 && n_decode <= 32 && n_splits > 1 && min(n_decode, 16) * n_splits <= 256 && hidden >= 16 &&
          hidden <= 2048;   // (wider: 28 heads of 128 at 3,584 +1%, 40 heads at 5,120 -0.5% with four tiles a wave)

@@ -127,6 +127,86 @@ __global__ __launch_bounds__(1024) void mlstm_step_kernel(MlstmArgs a, int lanes
   if (threadIdx.x == 0) a.maxima[size_t(slot) * a.heads + h] = m;
 }
 
+// The same for heads whose memory does not fit a block's registers: it passes through them for every token, NR rows of a group
+// at a time, the next rows on their way while these are used.
+template <typename T, int NR>
+__global__ __launch_bounds__(1024) void mlstm_stream_kernel(MlstmArgs a, int lanes) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];      // o [2][vdim]
+  __shared__ float scratch[16];
+  const int s = blockIdx.x, h = blockIdx.y, D = a.dim, V = a.vdim, threads = blockDim.x, R = threads / lanes;
+  const int group = threadIdx.x / lanes, l = threadIdx.x % lanes, d0 = 4 * l;
+  const bool in = d0 < D;
+  const int start = a.q_start[s], n = a.q_len[s], slot = a.state_slots[s];
+  float* kept = a.memory + (size_t(slot) * a.heads + h) * size_t(V + 1) * D + (in ? d0 : 0);
+  const float4 zero = make_float4(0.f, 0.f, 0.f, 0.f);
+  float4 norm = in ? load_four(kept + size_t(V) * D) : zero;
+  float m = a.maxima[size_t(slot) * a.heads + h];
+  const float q_scale = 1.0f / sqrtf(float(D)), bias_i = a.bias_i[h], bias_f = a.bias_f[h];
+  T* out = (T*)a.out;
+  for (int t = start; t < start + n; ++t) {
+    const T* row = (const T*)a.proj + size_t(t) * a.stride;
+    float4 S[NR], next[NR];
+    float value[NR], next_value[NR];
+    auto ask = [&](float4 (&rows)[NR], float (&values)[NR], int first) __attribute__((always_inline)) {
+#pragma unroll
+      for (int r = 0; r < NR; ++r) {      // always a valid address; what is past the end is not used
+        const int v = min(first + group + r * R, V - 1);
+        rows[r] = load_four(kept + size_t(v) * D);
+        values[r] = to_float(row[a.v_off + h * V + v]);
+      }
+    };
+    ask(S, value, 0);
+    const float i = log_input_gate(to_float(row[a.i_off + h]), bias_i, a.cap);
+    const float f = log_forget_gate(to_float(row[a.f_off + h]), bias_f, a.cap);
+    const float4 q = in ? load_four(row + a.q_off + h * D + d0) : zero, k = in ? load_four(row + a.k_off + h * D + d0) : zero;
+    const float top = fmaxf(f + m, i), keep = expf(f + m - top), take = expf(i - top);
+    m = top;
+    norm = make_float4(fmaf(keep, norm.x, take * k.x), fmaf(keep, norm.y, take * k.y), fmaf(keep, norm.z, take * k.z),
+                       fmaf(keep, norm.w, take * k.w));
+    float nq = dot4(norm, q);
+    for (int off = lanes >> 1; off > 0; off >>= 1) nq += __shfl_xor(nq, off, 64);
+    const float share = q_scale / (fmaxf(fabsf(nq * q_scale), expf(-m)) + kShareFloor);
+    float* o_row = lds + ((t - start) & 1) * V;
+    float squares = 0.f;
+    for (int first = 0; first < V; first += R * NR) {
+      const bool more = first + R * NR < V;
+      if (more) ask(next, next_value, first + R * NR);
+      float o[NR];
+#pragma unroll
+      for (int r = 0; r < NR; ++r) {
+        const int v = first + group + r * R;
+        const float tv = take * value[r];
+        const float4 x = make_float4(fmaf(keep, S[r].x, tv * k.x), fmaf(keep, S[r].y, tv * k.y), fmaf(keep, S[r].z, tv * k.z),
+                                     fmaf(keep, S[r].w, tv * k.w));
+        o[r] = in ? dot4(x, q) : 0.f;
+        if (in && v < V) *reinterpret_cast<float4*>(kept + size_t(v) * D) = x;
+      }
+      for (int off = lanes >> 1; off > 0; off >>= 1)
+#pragma unroll
+        for (int r = 0; r < NR; ++r) o[r] += __shfl_xor(o[r], off, 64);
+      if (l == 0) {
+#pragma unroll
+        for (int r = 0; r < NR; ++r) {
+          const int v = first + group + r * R;
+          const float x = o[r] * share;
+          if (v < V) { o_row[v] = x; squares = fmaf(x, x, squares); }
+        }
+      }
+      if (more) {
+#pragma unroll
+        for (int r = 0; r < NR; ++r) { S[r] = next[r]; value[r] = next_value[r]; }
+      }
+    }
+    squares = block_sum(squares, scratch);      // (its barriers also publish o_row)
+    const float unit = 1.0f / sqrtf(squares / float(V) + a.eps);
+    for (int v = threadIdx.x; v < V; v += threads)
+      out[(size_t(t) * a.heads + h) * V + v] =
+          from_float<T>(((o_row[v] * unit) * a.norm[h * V + v]) * sigmoid(to_float(row[a.gate_off + h * V + v])));
+  }
+  if (in && group == 0) *reinterpret_cast<float4*>(kept + size_t(V) * D) = norm;
+  if (threadIdx.x == 0) a.maxima[size_t(slot) * a.heads + h] = m;
+}
+
 // Any sizes: the memory stays in memory, a wave a row (the normaliser is row vdim, with the value one).
 template <typename T>
 __global__ __launch_bounds__(256) void mlstm_general_kernel(MlstmArgs a) {
@@ -564,7 +644,8 @@ static int launch_mlstm_chunks(hipStream_t s, const MlstmArgs& a, int T, int n_s
   return check_launch("sp_mlstm (chunks)");
 }
 
-// How a block of the step kernel holds a head's memory: lanes to a row, threads, rows a thread (0: it does not fit).
+// How a block of the step kernel holds a head's memory: lanes to a row, threads, rows a thread (0: no such kernel takes it; more
+// than 8: it passes through the registers).
 struct StepShape { int lanes, threads, rows; };
 static StepShape mlstm_step_shape(int dim, int vdim) {
   StepShape shape = {1, 256, 0};
@@ -573,7 +654,7 @@ static StepShape mlstm_step_shape(int dim, int vdim) {
   for (shape.threads = 256; shape.threads < 1024; shape.threads *= 2)
     if (vdim * shape.lanes <= 8 * shape.threads) break;
   const int R = shape.threads / shape.lanes, rows = (vdim + R - 1) / R;
-  shape.rows = rows <= 1 ? 1 : rows <= 2 ? 2 : rows <= 4 ? 4 : rows <= 8 ? 8 : rows <= 16 ? 16 : 0;
+  shape.rows = rows <= 1 ? 1 : rows <= 2 ? 2 : rows <= 4 ? 4 : rows <= 8 ? 8 : 16;
   return shape;
 }
 
@@ -586,7 +667,7 @@ static int launch_mlstm_step(hipStream_t s, const MlstmArgs& a, int n_seqs, Step
     case 2: mlstm_step_kernel<T, 2><<<grid, shape.threads, lds, s>>>(a, shape.lanes); break;
     case 4: mlstm_step_kernel<T, 4><<<grid, shape.threads, lds, s>>>(a, shape.lanes); break;
     case 8: mlstm_step_kernel<T, 8><<<grid, shape.threads, lds, s>>>(a, shape.lanes); break;
-    default: mlstm_step_kernel<T, 16><<<grid, shape.threads, lds, s>>>(a, shape.lanes); break;
+    default: mlstm_stream_kernel<T, 4><<<grid, shape.threads, lds, s>>>(a, shape.lanes); break;
   }
   return check_launch("sp_mlstm");
 }

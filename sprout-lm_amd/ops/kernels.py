@@ -82,7 +82,7 @@ def variant_code(table: dict, name: str, what: str) -> int:
 
 def check_attention_sizes(heads: int, kv_heads: int, head_dim: int) -> None:
     """Raises KernelError unless some attention kernel takes these sizes (any page size goes with them).
-    Head sizes of 16 ... 96 in steps of 16 and 128 run on the matrix cores in bfloat16, float32 in steps of 16 up
+    Head sizes of 16 ... 96 in steps of 16, 128, 160, 192 and 256 run on the matrix cores in bfloat16, float32 in steps of 16 up
     to 256 on the matrix cores' float32 instructions, every other size up to 512 on the general kernel."""
     if kv_heads <= 0 or heads <= 0 or heads % kv_heads:
         raise KernelError(f"attention: {heads} query heads do not divide into {kv_heads} key/value heads")

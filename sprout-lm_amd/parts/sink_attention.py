@@ -12,17 +12,17 @@ from ..weights.loader import TensorSpec
 from .base import Mixer, register_part
 
 # the head sizes the matrix-core attention kernels take; a head is kept this wide in the cache, zeros behind
-_KERNEL_WIDTHS = (16, 32, 48, 64, 80, 96, 128)
+_KERNEL_WIDTHS = (16, 32, 48, 64, 80, 96, 128, 160, 192, 256)
 
 
 def padded_width(dim: int, vdim: int) -> int:
     """The width at which keys and values of `dim` and `vdim` numbers are both kept: the next head size the
-    matrix-core kernels take, else the next multiple of 16 (float32 matrix cores up to 256), else as it is."""
+    matrix-core kernels take, else as it is."""
     need = max(dim, vdim)
     for width in _KERNEL_WIDTHS:
         if need <= width:
             return width
-    return -(-need // 16) * 16 if need <= 256 else need
+    return need
 
 
 @register_part("mixer", "sink_attention")
