@@ -229,8 +229,8 @@ PRESETS.update({
     # medium: latents of 128 + 64, memories of 8 heads of 128 x 256
     "varunex-m": _varunex_preset(2048, 12, 16, 2, 64, (16, 128, 64, 768, 128), (8, 128, 256), 4224, 32768),
     "varunex-m-twin": _morarax_preset(2048, 12, 16, 2, 128, 16, 16, 4224, 32768),
-    # large: latents of 192 + 64, memories of 8 heads of 256 x 512
-    "varunex-l": _varunex_preset(4096, 8, 32, 4, 64, (32, 128, 64, 1536, 192), (8, 256, 512), 8192, 32768),
+    # large: latents of 128 + 64, memories of 8 heads of 256 x 512
+    "varunex-l": _varunex_preset(4096, 8, 32, 4, 64, (32, 128, 64, 1536, 128), (8, 256, 512), 8192, 32768),
     "varunex-l-twin": _morarax_preset(4096, 8, 32, 4, 128, 32, 16, 8192, 32768),
 })
 

@@ -60,6 +60,18 @@ template <int DT>
 struct KVStep {
   bf16x8 ka[2][(DT + 1) / 2];   // K rows: tile of 16 keys x chunks of 32 dims
   uint2 va[DT][2];              // V^T rows: 16 dims x (4 keys of tile 0, 4 keys of tile 1)
+  static constexpr bool kLate = false;
+  __device__ __forceinline__ bf16x8 key(int kt, int c) const { return ka[kt][c]; }
+  __device__ __forceinline__ bf16x8 value(int dt) const { return as_bf16x8(make_uint4(va[dt][0].x, va[dt][0].y, va[dt][1].x, va[dt][1].y)); }
+};
+
+// A step that lies in LDS and is read operand by operand where it is used: wide heads have no registers to hold it in.  keys: this lane's first key row (the second tile's 16 rows on), values: its first value row (the next 16 rows on).
+template <int DT, int KP, int VP>
+struct LdsStep {
+  const uint16_t *keys, *values;
+  static constexpr bool kLate = true;
+  __device__ __forceinline__ bf16x8 key(int kt, int c) const { return as_bf16x8(*reinterpret_cast<const uint4*>(keys + 16 * kt * KP + 32 * c)); }
+  __device__ __forceinline__ bf16x8 value(int dt) const { return as_bf16x8(*reinterpret_cast<const uint4*>(values + 16 * dt * VP)); }
 };
 
 // Requests the 32 keys starting at key0 (a multiple of 32).  Loads are clamped to keys in [k_lo, k_hi];
@@ -166,8 +178,8 @@ __device__ __forceinline__ float fast_tanh(float x) {
 
 // qlo[qt]: the first key that this lane's row sees (first_visible of its position).
 // SIG: bias2 is the row's bias in log2 units (one query head a row), the weights are 1 / (1 + 2^-(s scale2 + bias2)).
-template <int DT, int NQT, bool MASKED, bool LAZY, bool CONTIG, bool SIG>
-__device__ __forceinline__ void attend_step_impl(const KVStep<DT>& r, const bf16x8 (&qop)[NQT][(DT + 1) / 2],
+template <int DT, int NQT, bool MASKED, bool LAZY, bool CONTIG, bool SIG, typename STEP>
+__device__ __forceinline__ void attend_step_impl(const STEP& r, const bf16x8 (&qop)[NQT][(DT + 1) / 2],
                                                  floatx4 (&o)[NQT][DT], float (&m)[NQT], float (&lsum)[NQT],
                                                  int key0, int k_lo, const int (&qpos)[NQT], const int (&qlo)[NQT],
                                                  const StepRule& rule, float scale2, float bias2) {
@@ -175,14 +187,30 @@ __device__ __forceinline__ void attend_step_impl(const KVStep<DT>& r, const bf16
   const int lane = threadIdx.x & 63, lj = lane >> 4;
 
   floatx4 s[NQT][2];
+  if constexpr (STEP::kLate) {      // an operand serves all tiles of rows while it is there
 #pragma unroll
-  for (int kt = 0; kt < 2; ++kt)
+    for (int kt = 0; kt < 2; ++kt)
 #pragma unroll
-    for (int qt = 0; qt < NQT; ++qt) {
-      s[qt][kt] = floatx4{0.f, 0.f, 0.f, 0.f};
+      for (int qt = 0; qt < NQT; ++qt) s[qt][kt] = floatx4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int c = 0; c < HC; ++c) s[qt][kt] = mfma16(r.ka[kt][c], qop[qt][c], s[qt][kt]);
-    }
+    for (int c = 0; c < HC; ++c)
+#pragma unroll
+      for (int kt = 0; kt < 2; ++kt) {
+        const bf16x8 key = r.key(kt, c);
+#pragma unroll
+        for (int qt = 0; qt < NQT; ++qt) s[qt][kt] = mfma16(key, qop[qt][c], s[qt][kt]);
+      }
+    __builtin_amdgcn_sched_barrier(0);
+  } else {
+#pragma unroll
+    for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+      for (int qt = 0; qt < NQT; ++qt) {
+        s[qt][kt] = floatx4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int c = 0; c < HC; ++c) s[qt][kt] = mfma16(r.key(kt, c), qop[qt][c], s[qt][kt]);
+      }
+  }
   if (rule.cap_mul > 0.f) {      // the same in every lane
 #pragma unroll
     for (int qt = 0; qt < NQT; ++qt)
@@ -250,6 +278,7 @@ __device__ __forceinline__ void attend_step_impl(const KVStep<DT>& r, const bf16
       for (int dt = 0; dt < DT; ++dt) o[qt][dt] *= alpha;
     }
   }
+  uint4 weights[STEP::kLate ? NQT : 1];
 #pragma unroll
   for (int qt = 0; qt < NQT; ++qt) {
     const float mx = m[qt];
@@ -268,18 +297,29 @@ __device__ __forceinline__ void attend_step_impl(const KVStep<DT>& r, const bf16
     if (!SIG) lsum[qt] += sum;
     const uint4 pb = make_uint4(pack_bf16x2(p[0][0], p[0][1]), pack_bf16x2(p[0][2], p[0][3]),
                                 pack_bf16x2(p[1][0], p[1][1]), pack_bf16x2(p[1][2], p[1][3]));
+    if constexpr (STEP::kLate) {
+      weights[qt] = pb;
+    } else {
+#pragma unroll
+      for (int dt = 0; dt < DT; ++dt) o[qt][dt] = mfma16(r.value(dt), as_bf16x8(pb), o[qt][dt]);
+    }
+  }
+  if constexpr (STEP::kLate) {
+    __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) {
-      const uint4 a = make_uint4(r.va[dt][0].x, r.va[dt][0].y, r.va[dt][1].x, r.va[dt][1].y);
-      o[qt][dt] = mfma16(as_bf16x8(a), as_bf16x8(pb), o[qt][dt]);
+      const bf16x8 value = r.value(dt);
+#pragma unroll
+      for (int qt = 0; qt < NQT; ++qt) o[qt][dt] = mfma16(value, as_bf16x8(weights[qt]), o[qt][dt]);
     }
+    __builtin_amdgcn_sched_barrier(0);
   }
 }
 
 // `first_pos`: smallest position among the rows that exist; a step whose 32 keys all lie at or before
 // it (and inside [k_lo, ...) where all rows see the same first key) needs no masking.
-template <int DT, int NQT, bool SIG, bool LAZY = true, bool CONTIG = false>
-__device__ __forceinline__ void attend_step(const KVStep<DT>& r, const bf16x8 (&qop)[NQT][(DT + 1) / 2],
+template <int DT, int NQT, bool SIG, bool LAZY = true, bool CONTIG = false, typename STEP>
+__device__ __forceinline__ void attend_step(const STEP& r, const bf16x8 (&qop)[NQT][(DT + 1) / 2],
                                             floatx4 (&o)[NQT][DT], float (&m)[NQT], float (&lsum)[NQT], int key0,
                                             int k_lo, const int (&qpos)[NQT], const int (&qlo)[NQT],
                                             const StepRule& rule, float scale2, float bias2, int first_pos) {
@@ -593,17 +633,18 @@ __global__ __launch_bounds__(64 * WPT * HPB) void attention_prefill_staged_kerne
     }
     __syncthreads();
   };
-  // A stage that takes more registers than a wave has to spare (wide heads on four waves) travels in pieces of eight: no
+  // A stage that takes more registers than a wave has to spare (wide heads on four waves) travels piece by piece: no
   // register is held while the stage before is used.
   constexpr bool PIECES = HD > 128 && !AHEAD;
+  constexpr int PIECE = THREADS > 256 ? 4 : 8;
   auto bring = [&](int key0, auto in_lds) __attribute__((always_inline)) {
     const bool interior = key0 >= f_lo && key0 + kStageKeys - 1 <= f_hi;
     __syncthreads();
 #pragma unroll 1
-    for (int u0 = 0; u0 < PER_THREAD; u0 += 8) {
-      uint4 piece[8];
+    for (int u0 = 0; u0 < PER_THREAD; u0 += PIECE) {
+      uint4 piece[PIECE];
 #pragma unroll
-      for (int u = 0; u < 8; ++u) {
+      for (int u = 0; u < PIECE; ++u) {
         const int i = threadIdx.x + THREADS * (u0 + u);
         if (i < KCHUNKS) {
           const int r = i / (HD / 8), c = i % (HD / 8);
@@ -618,7 +659,7 @@ __global__ __launch_bounds__(64 * WPT * HPB) void attention_prefill_staged_kerne
         }
       }
 #pragma unroll
-      for (int u = 0; u < 8; ++u) {
+      for (int u = 0; u < PIECE; ++u) {
         const int i = threadIdx.x + THREADS * (u0 + u);
         if (i < KCHUNKS) {
           const int r = i / (HD / 8), c = i % (HD / 8);
@@ -633,13 +674,17 @@ __global__ __launch_bounds__(64 * WPT * HPB) void attention_prefill_staged_kerne
   };
   // this wave's keys of the stage that lies in LDS, 32 at a time
   auto use_stage = [&](int key0) __attribute__((always_inline)) {
-    // (a wave that takes whole stages takes their steps one after the other: unrolled, their operands would not fit)
-    constexpr int UNROLL = WPT == 1 ? 1 : WAVE_KEYS / 32;
-#pragma unroll UNROLL
+#pragma unroll
     for (int sub = 0; sub < WAVE_KEYS / 32; ++sub) {
       const int skey = WAVE_KEYS * wave + 32 * sub;
       const int wkey = key0 + skey;
       if (has_head && wkey <= k_hi && (wkey + 32 > k_lo || wkey < st.keep)) {
+        if constexpr (HD > 128) {
+          static_assert(HD <= 128 || HD % 32 == 0, "whole chunks of 32 dimensions");
+          const LdsStep<DT, KP, VP> r = {ks + (skey + lr) * KP + 8 * lj, vs + lr * VP + skey + 8 * lj};
+          attend_step<DT, NQT, SIG, true, true>(r, qop, o, m, lsum, wkey, k_lo, qpos, qlo, rule, scale2, bias2, pos0);
+          continue;
+        }
         KVStep<DT> r;
 #pragma unroll
         for (int kt = 0; kt < 2; ++kt)
@@ -1111,13 +1156,14 @@ static bool staged_prefill(int page_size) { return page_size >= 8 && (page_size 
 // four teams of four waves.  Above that the registers of 16 waves do not suffice: four teams of two waves
 // (each wave then takes 64 keys of a stage).  Three teams were slower than two or four at every size.
 // A portion of 2,048 tokens at a context of 32,768: 835 -> 472 us (14 heads of 64), 2,350 -> 1,470 us (28 of 128).
-// Head sizes above 128 (a latent beside its turned part): one wave a head, four heads a block, so that a stage, which takes
-// most of the LDS, still serves four heads; a group of fewer heads, or a head of 256 (whose sums alone take half of a wave's
-// registers): four waves a head, a head a block.
+// Head sizes above 128 (a latent beside its turned part, under many heads): four heads a block on two waves each, so that a
+// stage, which takes most of the LDS, serves four heads and a SIMD has two waves; at 256 two heads on two waves each (a wave's
+// sums alone take half of the registers it then has).
 struct StagedShape { int hpb, wpt; bool ahead; };
 static StagedShape staged_shape(int nq, int nkv, int hd, int n_tiles) {
   const int G = nq / nkv;
-  if (hd > 128) return G >= 3 && hd <= 192 ? StagedShape{4, 1, false} : StagedShape{1, 4, false};
+  if (hd > 192) return G >= 2 ? StagedShape{2, 2, false} : StagedShape{1, 4, false};
+  if (hd > 128) return G >= 3 ? StagedShape{4, 2, false} : StagedShape{1, 4, false};
   if (G <= 1) return {1, 4, false};
   if (G == 2) return {2, 4, hd > 64};
   if (hd > 64) return {4, 2, false};
@@ -1186,7 +1232,8 @@ static int launch_mfma(hipStream_t s, const void* q, int q_stride, const void* k
       part_ml, splits, per_split, nq, nkv, page_shift, num_pages, st, scale2, n_tiles)
       // the same cases as staged_shape() and staged_paired()
       if constexpr (DT > 8) {
-        if (DT <= 12 && shape.hpb == 4) { if (paired) SP_STAGED(DT <= 12 ? 4 : 1, DT <= 12 ? 1 : 4, false, true); else SP_STAGED(DT <= 12 ? 4 : 1, DT <= 12 ? 1 : 4, false, false); }
+        constexpr int kHeads = DT > 12 ? 2 : 4;
+        if (shape.hpb == kHeads) { if (paired) SP_STAGED(kHeads, 2, false, true); else SP_STAGED(kHeads, 2, false, false); }
         else { if (paired) SP_STAGED(1, 4, false, true); else SP_STAGED(1, 4, false, false); }
       } else if (paired) {
         if (shape.hpb == 1) SP_STAGED(1, 4, false, true);
