@@ -56,8 +56,6 @@ int attention_mfma(hipStream_t s, const void* q, int q_stride, const void* k_poo
                                  page_size, num_pages, st, scale);
   }
 #undef SP_MFMA
-  set_error("sp_attention: no matrix-core kernel for head size %d", hd);
-  return 1;
 }
 
 // Decode steps whose chunks' merge is folded into the output projection.  Worth it where the merged partial

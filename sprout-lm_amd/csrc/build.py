@@ -20,7 +20,8 @@ FLAGS = ["-O3", "-std=c++17", "-fPIC", f"--offload-arch={ARCH}", "-Xclang", "-ta
 # Attention rescales its MFMA accumulators with vector instructions at every step, and so does the delta rule's state;
 # kept in AGPRs each such step would cost a move out and a move back, so these kernels take the VGPR form of MFMA.
 FILE_FLAGS = {name: ["-mllvm", "-amdgpu-mfma-vgpr-form"] for name in ("attention_mfma.hip", "attention_mfma_sigmoid.hip",
-                                                                              "attention_mfma_wide.hip", "delta.hip")}
+                                                                              "attention_mfma_wide.hip", "attention_mfma_wide_sigmoid.hip",
+                                                                              "delta.hip")}
 
 
 def sources() -> list[str]:

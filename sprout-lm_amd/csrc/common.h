@@ -64,6 +64,13 @@ __device__ __forceinline__ float gated_value(float g, float u, int act, float li
   return g / (1.0f + expf(-g)) * u;
 }
 
+// What a plain product's epilogue does to a number before it is stored: 0 = nothing, 1 = the square of max(x, 0).
+enum StoreAct : int { kStoreAsIs = 0, kStoreReluSquared = 1 };
+__device__ __forceinline__ float stored_value(float v, int act) {
+  if (act == kStoreReluSquared) { v = fmaxf(v, 0.f); v *= v; }
+  return v;
+}
+
 // Which earlier keys a query sees, and what stands between q . k and a key's weight.
 struct ScoreStage {
   int window;          // > 0: keys with position - key < window

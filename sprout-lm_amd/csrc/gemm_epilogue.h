@@ -19,7 +19,8 @@ struct RopeArgs {
   uint16_t* v_pool;              // [page][kv head][dim][slot]
   int nq, nkv, hd, page_size;
   const float2* table;           // [T][hd / 2] (cosine, sine) of positions[t] * inv_freq[d], or null: computed here
-  // the gated epilogue (kSilu) reads only these: which activation (GateAct of common.h; 0 = SiLU) and its limit
+  // the gated epilogue (kSilu) reads only these: which activation (GateAct of common.h; 0 = SiLU) and its limit; the plain store
+  // of bfloat16 (kStore) reads act alone: what is done to a number before it is stored (StoreAct)
   int act;
   float limit;
   const float* row_gate;         // may be null: a token's row is also multiplied by sigmoid(row_gate[t * row_gate_stride])
@@ -204,6 +205,8 @@ __device__ __forceinline__ void tile_epilogue(floatx16 (&acc)[WM][WN], float* tu
         const bool whole = n + 4 <= N && (N & 3) == 0;
         if (MODE == kStore) {
           uint16_t* dst = reinterpret_cast<uint16_t*>(out) + o;
+#pragma unroll
+          for (int r = 0; r < 4; ++r) v[r] = stored_value(v[r], rope.act);
           if (whole) *reinterpret_cast<uint2*>(dst) = make_uint2(pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3]));
           else for (int r = 0; r < 4 && n + r < N; ++r) dst[r] = f32_to_bf16_bits(v[r]);
         } else if (MODE == kStoreF32) {

@@ -52,6 +52,7 @@ struct FusedArgs {
   uint16_t* v_pool;
   int nq, nkv, hd, page_size, rotary_dim;
   int page_shift;            // page_size == 1 << page_shift, or -1 where it is no power of two
+  // kEpiStore: what is done to a number before it is stored (StoreAct of common.h).
   // kEpiSilu: which gated activation (GateAct of common.h) and its limit; row_gate (may be null): a token's row is
   // also multiplied by sigmoid(row_gate[t * row_gate_stride]), float32
   int act;
@@ -421,7 +422,7 @@ __global__ __launch_bounds__(256) void gemm_fused_kernel(FusedArgs a) {
         if (tp >= a.T || n >= a.N) continue;
         const float v = summed_at(pr >> 4, pr & 15, tn, token) + param_value(bias_bits[0], a.bias_bf16);
         const size_t o = size_t(tp) * a.N + n;
-        if (EPI == kEpiStore) reinterpret_cast<uint16_t*>(a.out)[o] = f32_to_bf16_bits(v);
+        if (EPI == kEpiStore) reinterpret_cast<uint16_t*>(a.out)[o] = f32_to_bf16_bits(stored_value(v, a.act));
         else if (EPI == kEpiStoreF32) reinterpret_cast<float*>(a.out)[o] = v;
         else if (gridDim.y == 1) reinterpret_cast<float*>(a.out)[o] += v;
         else unsafeAtomicAdd(reinterpret_cast<float*>(a.out) + o, v);
@@ -662,6 +663,29 @@ extern "C" int sp_gemm_decode(void* stream, const void* x, const float* residual
   if (mode == kEpiStore) return fused_norm<kEpiStore>(s, a, residual != nullptr, blocks, splits);
   if (mode == kEpiAccumulate) return fused_norm<kEpiAccumulate>(s, a, residual != nullptr, blocks, splits);
   return fused_norm<kEpiStoreF32>(s, a, residual != nullptr, blocks, splits);
+}
+
+// out (bfloat16) = act(x . w^T), act as StoreAct numbers it, in the product's own epilogue.
+extern "C" int sp_gemm_activated_takes(int T, int N, int K) {
+  return T <= 64 ? fused_shape_ok(T, K, false) && (N + 15) / 16 < 2048 : gemm_pipe_takes(T, N, K);
+}
+
+namespace sprout {
+int gemm_bf16_pipe_activated(hipStream_t s, const void* a, const void* w, int act, void* out, int T, int N, int K);
+}
+
+extern "C" int sp_gemm_activated(void* stream, const void* x, const void* w, int act, void* out, int T, int N, int K) {
+  SP_REQUIRE(act == kStoreReluSquared, "sp_gemm_activated: no activation %d (1 = the square of ReLU)", act);
+  SP_REQUIRE(T > 0 && N > 0 && K > 0 && sp_gemm_activated_takes(T, N, K), "sp_gemm_activated: shape T=%d N=%d K=%d is not taken", T, N, K);
+  SP_REQUIRE(x && w && out && ((reinterpret_cast<uintptr_t>(x) | reinterpret_cast<uintptr_t>(w)) & 15) == 0,
+             "sp_gemm_activated: operands must start at a multiple of 16 bytes");
+  hipStream_t s = (hipStream_t)stream;
+  if (T > 64) return gemm_bf16_pipe_activated(s, x, w, act, out, T, N, K);
+  FusedArgs a = {};
+  a.x = (const uint16_t*)x; a.w = (const uint16_t*)w; a.out = out; a.act = act;
+  a.T = T; a.N = N; a.K = K;
+  a.k_per_split = (K + 63) / 64 * 64;
+  return fused_norm<kEpiStore>(s, a, false, (N + 31) / 32, 1);
 }
 
 // q/k/v projection with bias, rotation and cache write.  w is [(nq + 2 nkv) * hd, K] (q, k, v rows).

@@ -301,31 +301,31 @@ void pipe_choice(int T, int N, int K, bool may_split, int* shape, int* splits, b
 
 template <int WM, int WN, int WAVES_M, int WAVES_N, int STAGES, typename TB>
 inline int launch_pipe(hipStream_t s, const void* x, const void* w, const void* bias, int mode, void* out, int T, int N,
-                       int K, int splits) {
+                       int K, int splits, const RopeArgs& epilogue) {
   const int k_per_split = ((K / 64 + splits - 1) / splits) * 64;
   splits = (K + k_per_split - 1) / k_per_split;
   const uint16_t *xp = (const uint16_t*)x, *wp = (const uint16_t*)w;
   const TB* bp = (const TB*)bias;
-  if (mode == kStore) return launch_pipe_mode<WM, WN, WAVES_M, WAVES_N, STAGES, kStore, TB>(s, splits, xp, wp, bp, out, T, N, K, k_per_split);
+  if (mode == kStore) return launch_pipe_mode<WM, WN, WAVES_M, WAVES_N, STAGES, kStore, TB>(s, splits, xp, wp, bp, out, T, N, K, k_per_split, epilogue);
   if (mode == kAccumulate) return launch_pipe_mode<WM, WN, WAVES_M, WAVES_N, STAGES, kAccumulate, TB>(s, splits, xp, wp, bp, out, T, N, K, k_per_split);
   return launch_pipe_mode<WM, WN, WAVES_M, WAVES_N, STAGES, kStoreF32, TB>(s, splits, xp, wp, bp, out, T, N, K, k_per_split);
 }
 
 template <typename TB>
 inline int pipe_shape(hipStream_t s, const void* x, const void* w, const void* bias, int mode, void* out, int T, int N,
-                      int K) {
+                      int K, const RopeArgs& epilogue = RopeArgs{}) {
   int shape, splits;
   pipe_choice(T, N, K, mode == kAccumulate, &shape, &splits);
   switch (shape) {
-    case 0: return launch_pipe<4, 2, 2, 4, 2, TB>(s, x, w, bias, mode, out, T, N, K, splits);
-    case 1: return launch_pipe<2, 2, 4, 2, 3, TB>(s, x, w, bias, mode, out, T, N, K, splits);
-    case 2: return launch_pipe<1, 2, 4, 2, 4, TB>(s, x, w, bias, mode, out, T, N, K, splits);
-    case 4: return launch_pipe<1, 2, 2, 4, 3, TB>(s, x, w, bias, mode, out, T, N, K, splits);
-    case 5: return launch_pipe<1, 2, 2, 2, 3, TB>(s, x, w, bias, mode, out, T, N, K, splits);
-    case 6: return launch_pipe<6, 2, 2, 4, 2, TB>(s, x, w, bias, mode, out, T, N, K, splits);
-    case 7: return launch_pipe<1, 2, 2, 1, 4, TB>(s, x, w, bias, mode, out, T, N, K, splits);
-    case 8: return launch_pipe<2, 5, 4, 1, 3, TB>(s, x, w, bias, mode, out, T, N, K, splits);
-    default: return launch_pipe<1, 1, 2, 2, 4, TB>(s, x, w, bias, mode, out, T, N, K, splits);
+    case 0: return launch_pipe<4, 2, 2, 4, 2, TB>(s, x, w, bias, mode, out, T, N, K, splits, epilogue);
+    case 1: return launch_pipe<2, 2, 4, 2, 3, TB>(s, x, w, bias, mode, out, T, N, K, splits, epilogue);
+    case 2: return launch_pipe<1, 2, 4, 2, 4, TB>(s, x, w, bias, mode, out, T, N, K, splits, epilogue);
+    case 4: return launch_pipe<1, 2, 2, 4, 3, TB>(s, x, w, bias, mode, out, T, N, K, splits, epilogue);
+    case 5: return launch_pipe<1, 2, 2, 2, 3, TB>(s, x, w, bias, mode, out, T, N, K, splits, epilogue);
+    case 6: return launch_pipe<6, 2, 2, 4, 2, TB>(s, x, w, bias, mode, out, T, N, K, splits, epilogue);
+    case 7: return launch_pipe<1, 2, 2, 1, 4, TB>(s, x, w, bias, mode, out, T, N, K, splits, epilogue);
+    case 8: return launch_pipe<2, 5, 4, 1, 3, TB>(s, x, w, bias, mode, out, T, N, K, splits, epilogue);
+    default: return launch_pipe<1, 1, 2, 2, 4, TB>(s, x, w, bias, mode, out, T, N, K, splits, epilogue);
   }
 }
 

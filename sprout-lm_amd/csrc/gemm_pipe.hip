@@ -105,4 +105,11 @@ int gemm_bf16_pipe(hipStream_t s, const void* a, const void* w, int bias_dtype, 
   return pipe_shape<float>(s, a, w, bias, mode, out, T, N, K);
 }
 
+// The same with what StoreAct does to every number before it is stored (bfloat16, no bias).
+int gemm_bf16_pipe_activated(hipStream_t s, const void* a, const void* w, int act, void* out, int T, int N, int K) {
+  RopeArgs epilogue = {};
+  epilogue.act = act;
+  return pipe_shape<float>(s, a, w, nullptr, kStore, out, T, N, K, epilogue);
+}
+
 }  // namespace sprout

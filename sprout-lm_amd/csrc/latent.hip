@@ -4,7 +4,7 @@
 // latent in the same width (the value pool's columns behind the latent are never written and stay zero), so that every
 // attention kernel for one key/value head and heads of `width` takes it.  Queries for that attention are
 // [query . U_k (rank numbers, written by the per-head product), rotated part, zeros].  Up to three jobs a launch, a block a
-// token: norm the latent, turn the shared key part and cache both; turn every head's query part; norm a query latent.
+// token and job: norm the latent, turn the shared key part and cache both; turn every head's query part; norm a query latent.
 //
 // Rotation: the first rot_dims numbers of a rotated part turn, (2i, 2i + 1) or (i, i + rot_dims / 2) together, by
 // position * freq[i], and cosine and sine are multiplied by `magnitude`; the rest pass unchanged.  exact != 0: angle, sine
@@ -35,6 +35,7 @@ struct LatentArgs {
   int cq_stride, cq_off, cq_rank;
   const void* cq_norm;
   void* cq_out;
+  int jobs[3];                 // blockIdx.y: which job (0 the latent, 1 the queries, 2 the query latent)
 };
 
 // One over the root mean square of n numbers, over the whole block.
@@ -53,7 +54,8 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(LatentArgs a) {
   extern __shared__ float cs[];      // [rot_dims / 2][2] cosine, sine (times magnitude)
   __shared__ float scratch[16];
   const int t = blockIdx.x, rank = a.rank, rot = a.rot, width = a.width, pairs = a.rot_dims / 2;
-  if (a.kv || a.q) {
+  const int job = a.jobs[blockIdx.y];
+  if (job < 2 && a.rot_dims > 0) {
     const int pos = a.positions[t];
     for (int i = threadIdx.x; i < pairs; i += blockDim.x) {
       float c, s;
@@ -90,7 +92,7 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(LatentArgs a) {
     return second ? v * c + u * s : u * c - v * s;
   };
 
-  if (a.kv) {
+  if (job == 0) {
     const T* row = (const T*)a.kv + size_t(t) * a.kv_stride + a.kv_off;
     const TW* norm_w = (const TW*)a.kv_norm;
     const int slot = a.slot_mapping[t];
@@ -107,14 +109,14 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(LatentArgs a) {
       for (int d = threadIdx.x; d < width - rank; d += blockDim.x) key[rank + d] = from_float<T>(d < rot ? turned(row + rank, d) : 0.f);
     }
   }
-  if (a.cq) {
+  if (job == 2) {
     const T* row = (const T*)a.cq + size_t(t) * a.cq_stride + a.cq_off;
     const TW* norm_w = (const TW*)a.cq_norm;
     const float scale = unit_of(row, a.cq_rank, a.eps, scratch);
     T* out = (T*)a.cq_out + size_t(t) * a.cq_rank;
     for (int d = threadIdx.x; d < a.cq_rank; d += blockDim.x) out[d] = from_float<T>((to_float(row[d]) * scale) * to_float(norm_w[d]));
   }
-  if (a.q) {
+  if (job == 1) {
     const T* row = (const T*)a.q + size_t(t) * a.q_stride + a.q_off;
     T* out = (T*)a.q_out + size_t(t) * a.heads * width;
     const int tail = width - rank;
@@ -150,13 +152,18 @@ extern "C" int sp_latent_prepare(void* stream, int dtype, int heads, int dim, in
              "sp_latent_prepare: unsupported dtypes %d, %d", dtype, norm_w_dtype);
   if (T == 0 || (!kv && !q && !cq)) return 0;
   hipStream_t s = (hipStream_t)stream;
-  const LatentArgs a = {heads, dim, rot, rank, width, eps, positions, freq, rot_dims, magnitude, pairing, exact, kv, kv_stride, kv_off,
+  LatentArgs a = {heads, dim, rot, rank, width, eps, positions, freq, rot_dims, magnitude, pairing, exact, kv, kv_stride, kv_off,
                         kv_norm, slot_mapping, k_pool, v_pool, page_size, q, q_stride, q_off, q_out, cq, cq_stride, cq_off, cq_rank,
-                        cq_norm, cq_out};
+                        cq_norm, cq_out, {0, 0, 0}};
+  int n_jobs = 0;
+  if (kv) a.jobs[n_jobs++] = 0;
+  if (q) a.jobs[n_jobs++] = 1;
+  if (cq) a.jobs[n_jobs++] = 2;
+  const dim3 grid(T, n_jobs);
   const size_t lds = size_t(rot_dims > 0 ? rot_dims : 2) * sizeof(float);
-  if (dtype == kF32 && norm_w_dtype == kF32) latent_prepare_kernel<float, float><<<T, 256, lds, s>>>(a);
-  else if (dtype == kF32) latent_prepare_kernel<float, bf16_t><<<T, 256, lds, s>>>(a);
-  else if (norm_w_dtype == kF32) latent_prepare_kernel<bf16_t, float><<<T, 256, lds, s>>>(a);
-  else latent_prepare_kernel<bf16_t, bf16_t><<<T, 256, lds, s>>>(a);
+  if (dtype == kF32 && norm_w_dtype == kF32) latent_prepare_kernel<float, float><<<grid, 256, lds, s>>>(a);
+  else if (dtype == kF32) latent_prepare_kernel<float, bf16_t><<<grid, 256, lds, s>>>(a);
+  else if (norm_w_dtype == kF32) latent_prepare_kernel<bf16_t, float><<<grid, 256, lds, s>>>(a);
+  else latent_prepare_kernel<bf16_t, bf16_t><<<grid, 256, lds, s>>>(a);
   return check_launch("sp_latent_prepare");
 }

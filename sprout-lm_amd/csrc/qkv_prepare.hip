@@ -41,12 +41,29 @@ __device__ __forceinline__ float row_scale(const T* __restrict__ x, int n, float
   return 1.0f / sqrtf(block_sum(sq, scratch) / float(n) + eps);
 }
 
+// Cosine and sine (times magnitude) of pair d at the token's position.
+__device__ __forceinline__ float2 turn_of(const PrepareArgs& a, int t, int d) {
+  float sn, cs;
+  if (a.inv_freq_tail) {
+    double sn64, cs64;
+    sincos(double(a.positions[t]) * (double(a.inv_freq[d]) + double(a.inv_freq_tail[d])), &sn64, &cs64);
+    sn = float(sn64 * double(a.magnitude));
+    cs = float(cs64 * double(a.magnitude));
+  } else {
+    sincosf(float(a.positions[t]) * a.inv_freq[d], &sn, &cs);
+    sn *= a.magnitude;
+    cs *= a.magnitude;
+  }
+  return make_float2(cs, sn);
+}
+
+// `turns`: every pair's cosine and sine of this token, or null: computed here.
 // One head of one token (query heads, then key heads, then value heads), by `count` threads of which this is `lane`.
 // `scratch` (16 floats): where `count` is the whole block, the head's sum of squares is taken over it; otherwise the
 // head belongs to one wave.
 template <typename T>
 __device__ __forceinline__ void prepare_head(const PrepareArgs& a, int t, int head, float q_scale, float k_scale, int slot,
-                                             int lane, int count, float* scratch, bool whole_block) {
+                                             int lane, int count, float* scratch, bool whole_block, const float2* turns) {
   const T* row = (const T*)a.proj + size_t(t) * a.stride;
   const int nq = a.nq, nkv = a.nkv, nk = nkv * a.maps, D = a.dim, V = a.vdim, W = a.width;      // nk: rows of keys
   const int page = slot >= 0 ? slot / a.page_size : 0, off = slot >= 0 ? slot % a.page_size : 0;
@@ -101,20 +118,10 @@ __device__ __forceinline__ void prepare_head(const PrepareArgs& a, int t, int he
     if (d >= D) { dst[d] = from_float<T>(0.f); continue; }
     if (d >= 2 * half) { dst[d] = from_float<T>(normed(d) * unit); continue; }
     if (d >= half) continue;          // written by the owner of its pair
-    float sn, cs;
-    if (a.inv_freq_tail) {
-      double sn64, cs64;
-      sincos(double(a.positions[t]) * (double(a.inv_freq[d]) + double(a.inv_freq_tail[d])), &sn64, &cs64);
-      sn = float(sn64 * double(a.magnitude));
-      cs = float(cs64 * double(a.magnitude));
-    } else {
-      sincosf(float(a.positions[t]) * a.inv_freq[d], &sn, &cs);
-      sn *= a.magnitude;
-      cs *= a.magnitude;
-    }
+    const float2 turn = turns ? turns[d] : turn_of(a, t, d);
     const float x = normed(d), y = normed(d + half);
-    dst[d] = from_float<T>((x * cs - y * sn) * unit);
-    dst[d + half] = from_float<T>((y * cs + x * sn) * unit);
+    dst[d] = from_float<T>((x * turn.x - y * turn.y) * unit);
+    dst[d + half] = from_float<T>((y * turn.x + x * turn.y) * unit);
   }
 }
 
@@ -134,7 +141,7 @@ __device__ __forceinline__ float4 round4(float4 v) {
                      __uint_as_float(p.y & 0xffff0000u));
 }
 __device__ __forceinline__ void prepare_head_fours(const PrepareArgs& a, int t, int head, float q_scale, float k_scale, int slot,
-                                                   int lane, int count) {
+                                                   int lane, int count, const float2* turns) {
   const bf16_t* row = (const bf16_t*)a.proj + size_t(t) * a.stride;
   const int nq = a.nq, nkv = a.nkv, nk = nkv * a.maps, D = a.dim, V = a.vdim, W = a.width;
   const int page = slot >= 0 ? slot / a.page_size : 0, off = slot >= 0 ? slot % a.page_size : 0;
@@ -193,10 +200,15 @@ __device__ __forceinline__ void prepare_head_fours(const PrepareArgs& a, int t, 
     if (d >= D) { *reinterpret_cast<uint2*>(dst + d) = make_uint2(0u, 0u); continue; }
     if (d >= 2 * half) { *reinterpret_cast<uint2*>(dst + d) = pack4(normed(d)); continue; }
     if (d >= half) continue;
-    const float pos = float(a.positions[t]);
     float sn[4], cs[4];
+    if (turns) {
 #pragma unroll
-    for (int j = 0; j < 4; ++j) sincosf(pos * a.inv_freq[d + j], &sn[j], &cs[j]);
+      for (int j = 0; j < 4; ++j) { cs[j] = turns[d + j].x; sn[j] = turns[d + j].y; }
+    } else {
+      const float pos = float(a.positions[t]);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) sincosf(pos * a.inv_freq[d + j], &sn[j], &cs[j]);
+    }
     const float4 x = normed(d), y = normed(d + half);
     *reinterpret_cast<uint2*>(dst + d) = pack4(make_float4(x.x * cs[0] - y.x * sn[0], x.y * cs[1] - y.y * sn[1],
                                                            x.z * cs[2] - y.z * sn[2], x.w * cs[3] - y.w * sn[3]));
@@ -218,6 +230,8 @@ __device__ __forceinline__ float row_scale_fours(const bf16_t* __restrict__ x, i
   return 1.0f / sqrtf(block_sum(sq, scratch) / float(n) + eps);
 }
 
+constexpr int kTurnsInLds = 256;      // pairs of numbers that turn whose cosines and sines a block keeps
+
 // FOURS (bfloat16 only): every size is in fours and every row starts at a multiple of 8 bytes.
 template <typename T, bool PER_HEAD, bool FOURS>
 __global__ __launch_bounds__(256) void qkv_prepare_kernel(PrepareArgs a) {
@@ -235,9 +249,17 @@ __global__ __launch_bounds__(256) void qkv_prepare_kernel(PrepareArgs a) {
       if constexpr (FOURS) scale = row_scale_fours(whole, n, a.eps, scratch);
       else scale = row_scale(whole, n, a.eps, scratch);
     }
-    if constexpr (FOURS) prepare_head_fours(a, t, head, scale, scale, slot, threadIdx.x, blockDim.x);
-    else prepare_head<T>(a, t, head, scale, scale, slot, threadIdx.x, blockDim.x, scratch, true);
+    if constexpr (FOURS) prepare_head_fours(a, t, head, scale, scale, slot, threadIdx.x, blockDim.x, nullptr);
+    else prepare_head<T>(a, t, head, scale, scale, slot, threadIdx.x, blockDim.x, scratch, true, nullptr);
     return;
+  }
+  // the token's cosines and sines, once for all its heads
+  __shared__ float2 turns[PER_HEAD ? 1 : kTurnsInLds];
+  const int pairs = a.rotary_dim / 2;
+  const bool kept = pairs > 0 && pairs <= kTurnsInLds;
+  if (kept) {
+    for (int d = threadIdx.x; d < pairs; d += blockDim.x) turns[d] = turn_of(a, t, d);
+    __syncthreads();
   }
   float q_scale = 1.f, k_scale = 1.f;
   if (a.q_norm) {
@@ -251,8 +273,8 @@ __global__ __launch_bounds__(256) void qkv_prepare_kernel(PrepareArgs a) {
   }
   const int wave = threadIdx.x >> 6, waves = blockDim.x >> 6;
   for (int head = wave; head < heads; head += waves) {
-    if constexpr (FOURS) prepare_head_fours(a, t, head, q_scale, k_scale, slot, threadIdx.x & 63, 64);
-    else prepare_head<T>(a, t, head, q_scale, k_scale, slot, threadIdx.x & 63, 64, scratch, false);
+    if constexpr (FOURS) prepare_head_fours(a, t, head, q_scale, k_scale, slot, threadIdx.x & 63, 64, kept ? turns : nullptr);
+    else prepare_head<T>(a, t, head, q_scale, k_scale, slot, threadIdx.x & 63, 64, scratch, false, kept ? turns : nullptr);
   }
 }
 

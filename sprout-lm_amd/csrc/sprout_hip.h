@@ -45,6 +45,9 @@ int sp_pipe_plan(int kind, int T, int N, int K, int hd, int* plan);
 int sp_pipe_tiles(int tiles_t, int tiles_n, int* tile_of, int room);
 int sp_gemm_decode(void* stream, const void* x, const float* residual, int norm_w_dtype, const void* norm_w, float eps,
                    const void* w, int bias_dtype, const void* bias, int mode, void* out, int T, int N, int K);
+// out [T, N] (bfloat16) = act(x . w^T) with the activation in the product's epilogue, act 1 = max(v, 0)^2; bfloat16 operands.
+int sp_gemm_activated_takes(int T, int N, int K);
+int sp_gemm_activated(void* stream, const void* x, const void* w, int act, void* out, int T, int N, int K);
 // q, k, v projection (+ bias), rotation of q and k, q to q_out [T, nq * hd], k and v into the paged pools.
 // With more than 64 tokens (head sizes that are multiples of 64) the tiled product does it in its epilogue;
 // cos_sin (may be null): the table of sp_rope_table for these positions, which saves it the sines and cosines.

@@ -1033,6 +1033,25 @@ def activation(x: torch.Tensor, kind: str) -> None:
                                   variant_code(UNARY_ACTIVATIONS, kind, "activation")))
 
 
+FOLDED_ACTIVATIONS = {"relu_squared": 1}      # unary activations that the plain product has in its epilogue
+
+
+def gemm_activated(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, kind: str) -> bool:
+    """out = act(x . w^T) in one kernel (bfloat16, no bias).  Returns False (and does nothing) where no product kernel has the
+    activation in its epilogue for the call; the caller then multiplies and activates in turn."""
+    act = FOLDED_ACTIVATIONS.get(kind)
+    if act is None or x.dtype != torch.bfloat16 or w.dtype != torch.bfloat16 or out.dtype != torch.bfloat16:
+        return False
+    T, (N, K) = x.shape[0], w.shape
+    if x.shape[1] != K or tuple(out.shape) != (T, N) or not (x.is_contiguous() and w.is_contiguous() and out.is_contiguous()):
+        raise KernelError(f"gemm_activated: shapes do not fit: x {tuple(x.shape)}, w {tuple(w.shape)}, out {tuple(out.shape)}")
+    if T == 0 or K % 8 or (x.data_ptr() | w.data_ptr()) & 15 or not library().sp_gemm_activated_takes(T, N, K):
+        return False
+    _gpu(x, "input"); _gpu(w, "weight"); _gpu(out, "output")
+    check(library().sp_gemm_activated(_stream(), x.data_ptr(), w.data_ptr(), act, out.data_ptr(), T, N, K))
+    return True
+
+
 def scale_rows(x: torch.Tensor, weights: torch.Tensor, out: torch.Tensor) -> None:
     """out[t * top + k] = x[t] * weights[t, k]: a token's row once per choice, times the choice's weight."""
     _gpu(x, "rows"); _gpu(weights, "row weights"); _gpu(out, "scaled rows")

@@ -36,6 +36,8 @@ def _declare(lib):
         "sp_pipe_tiles": [c_int, c_int, ctypes.POINTER(c_int), c_int],
         "sp_gemm_decode": [c_void, c_void, c_void, c_int, c_void, c_float, c_void, c_int, c_void, c_int, c_void, c_int,
                            c_int, c_int],
+        "sp_gemm_activated_takes": [c_int] * 3,
+        "sp_gemm_activated": [c_void, c_void, c_void, c_int, c_void, c_int, c_int, c_int],
         "sp_qkv_rope_cache": [c_void, c_void, c_void, c_int, c_void, c_float, c_void, c_int, c_void, c_void, c_void,
                               c_void, c_int, c_void, c_void, c_void, c_int, c_int, c_int, c_int, c_int, c_int, c_void, c_int],
         "sp_rope_table": [c_void, c_void, c_void, c_void, c_int, c_float, c_void, c_int],

@@ -144,6 +144,7 @@ class DenseMLP(FeedForward):
     def forward(self, ctx, h, residual):
         T = h.shape[0]
         act = ctx.buffer("mlp_inner", (T, self.inner), ctx.act_dtype)
-        ops.gemm(h, self.w_up, act, bias=self.b_up)
-        ops.activation(act, self.activation)
+        if self.b_up is not None or not ops.gemm_activated(h, self.w_up, act, self.activation):
+            ops.gemm(h, self.w_up, act, bias=self.b_up)
+            ops.activation(act, self.activation)
         ops.gemm(act, self.w_down, residual, bias=self.b_down, accumulate=True)
