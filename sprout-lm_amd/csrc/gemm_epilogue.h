@@ -19,12 +19,17 @@ struct RopeArgs {
   uint16_t* v_pool;              // [page][kv head][dim][slot]
   int nq, nkv, hd, page_size;
   const float2* table;           // [T][hd / 2] (cosine, sine) of positions[t] * inv_freq[d], or null: computed here
-  // the gated epilogue (kSilu) reads only these: which activation (GateAct of common.h; 0 = SiLU) and its limit; the plain store
-  // of bfloat16 (kStore) reads act alone: what is done to a number before it is stored (StoreAct)
+  // the gated epilogue (kSilu) reads only these: which activation (GateAct of common.h; 0 = SiLU) and its limit
   int act;
   float limit;
   const float* row_gate;         // may be null: a token's row is also multiplied by sigmoid(row_gate[t * row_gate_stride])
   long long row_gate_stride;
+  // the plain store of bfloat16 (kStore): where `second` is given, weight rows from `split` on are a product of their own: what
+  // `act` (StoreAct) makes of them goes to second[t * second_stride + n - split], the others to out[t * out_stride + n]; split and
+  // strides in fours
+  uint16_t* second;
+  int split;
+  long long out_stride, second_stride;
 };
 
 // Orders a wave's LDS writes before its own later reads of what other lanes wrote (and the reverse).
@@ -205,8 +210,15 @@ __device__ __forceinline__ void tile_epilogue(floatx16 (&acc)[WM][WN], float* tu
         const bool whole = n + 4 <= N && (N & 3) == 0;
         if (MODE == kStore) {
           uint16_t* dst = reinterpret_cast<uint16_t*>(out) + o;
+          if (rope.second) {
+            if (n >= rope.split) {
+              dst = rope.second + size_t(t) * rope.second_stride + (n - rope.split);
 #pragma unroll
-          for (int r = 0; r < 4; ++r) v[r] = stored_value(v[r], rope.act);
+              for (int r = 0; r < 4; ++r) v[r] = stored_value(v[r], rope.act);
+            } else {
+              dst = reinterpret_cast<uint16_t*>(out) + size_t(t) * rope.out_stride + n;
+            }
+          }
           if (whole) *reinterpret_cast<uint2*>(dst) = make_uint2(pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3]));
           else for (int r = 0; r < 4 && n + r < N; ++r) dst[r] = f32_to_bf16_bits(v[r]);
         } else if (MODE == kStoreF32) {

@@ -52,7 +52,10 @@ struct FusedArgs {
   uint16_t* v_pool;
   int nq, nkv, hd, page_size, rotary_dim;
   int page_shift;            // page_size == 1 << page_shift, or -1 where it is no power of two
-  // kEpiStore: what is done to a number before it is stored (StoreAct of common.h).
+  // kEpiStore: a second product of the same input in the weight rows from `split` on (null: none), as RopeArgs describes it
+  uint16_t* second;
+  int split;
+  long long out_stride, second_stride;
   // kEpiSilu: which gated activation (GateAct of common.h) and its limit; row_gate (may be null): a token's row is
   // also multiplied by sigmoid(row_gate[t * row_gate_stride]), float32
   int act;
@@ -422,7 +425,19 @@ __global__ __launch_bounds__(256) void gemm_fused_kernel(FusedArgs a) {
         if (tp >= a.T || n >= a.N) continue;
         const float v = summed_at(pr >> 4, pr & 15, tn, token) + param_value(bias_bits[0], a.bias_bf16);
         const size_t o = size_t(tp) * a.N + n;
-        if (EPI == kEpiStore) reinterpret_cast<uint16_t*>(a.out)[o] = f32_to_bf16_bits(stored_value(v, a.act));
+        if (EPI == kEpiStore) {
+          uint16_t* dst = reinterpret_cast<uint16_t*>(a.out) + o;
+          float stored = v;
+          if (a.second) {
+            if (n >= a.split) {
+              dst = a.second + size_t(tp) * a.second_stride + (n - a.split);
+              stored = stored_value(v, a.act);
+            } else {
+              dst = reinterpret_cast<uint16_t*>(a.out) + size_t(tp) * a.out_stride + n;
+            }
+          }
+          *dst = f32_to_bf16_bits(stored);
+        }
         else if (EPI == kEpiStoreF32) reinterpret_cast<float*>(a.out)[o] = v;
         else if (gridDim.y == 1) reinterpret_cast<float*>(a.out)[o] += v;
         else unsafeAtomicAdd(reinterpret_cast<float*>(a.out) + o, v);
@@ -665,24 +680,31 @@ extern "C" int sp_gemm_decode(void* stream, const void* x, const float* residual
   return fused_norm<kEpiStoreF32>(s, a, residual != nullptr, blocks, splits);
 }
 
-// out (bfloat16) = act(x . w^T), act as StoreAct numbers it, in the product's own epilogue.
-extern "C" int sp_gemm_activated_takes(int T, int N, int K) {
+// Two products of the same input in one: rows 0 .. split - 1 of w to out, what act makes of the others to second.
+extern "C" int sp_gemm_joined_takes(int T, int N, int K) {
   return T <= 64 ? fused_shape_ok(T, K, false) && (N + 15) / 16 < 2048 : gemm_pipe_takes(T, N, K);
 }
 
 namespace sprout {
-int gemm_bf16_pipe_activated(hipStream_t s, const void* a, const void* w, int act, void* out, int T, int N, int K);
+int gemm_bf16_pipe_joined(hipStream_t s, const void* a, const void* w, const float* bias, int act, void* out, long long out_stride,
+                          int split, void* second, long long second_stride, int T, int N, int K);
 }
 
-extern "C" int sp_gemm_activated(void* stream, const void* x, const void* w, int act, void* out, int T, int N, int K) {
-  SP_REQUIRE(act == kStoreReluSquared, "sp_gemm_activated: no activation %d (1 = the square of ReLU)", act);
-  SP_REQUIRE(T > 0 && N > 0 && K > 0 && sp_gemm_activated_takes(T, N, K), "sp_gemm_activated: shape T=%d N=%d K=%d is not taken", T, N, K);
-  SP_REQUIRE(x && w && out && ((reinterpret_cast<uintptr_t>(x) | reinterpret_cast<uintptr_t>(w)) & 15) == 0,
-             "sp_gemm_activated: operands must start at a multiple of 16 bytes");
+extern "C" int sp_gemm_joined(void* stream, const void* x, const void* w, const float* bias, int act, void* out,
+                              long long out_stride, int split, void* second, long long second_stride, int T, int N, int K) {
+  SP_REQUIRE(act == kStoreAsIs || act == kStoreReluSquared, "sp_gemm_joined: no activation %d (1 = the square of ReLU)", act);
+  SP_REQUIRE(T > 0 && N > 0 && K > 0 && sp_gemm_joined_takes(T, N, K), "sp_gemm_joined: shape T=%d N=%d K=%d is not taken", T, N, K);
+  SP_REQUIRE(split >= 0 && split < N && split % 4 == 0 && N % 4 == 0 && out_stride % 4 == 0 && second_stride % 4 == 0 &&
+                 out_stride >= split && second_stride >= N - split,
+             "sp_gemm_joined: %d and %d rows do not go to rows of %lld and %lld numbers", split, N - split, out_stride, second_stride);
+  SP_REQUIRE(x && w && second && (out || split == 0) && ((reinterpret_cast<uintptr_t>(x) | reinterpret_cast<uintptr_t>(w)) & 15) == 0 &&
+                 ((reinterpret_cast<uintptr_t>(out) | reinterpret_cast<uintptr_t>(second)) & 7) == 0,
+             "sp_gemm_joined: null operand, or one that does not start at a multiple of 16 (8: results) bytes");
   hipStream_t s = (hipStream_t)stream;
-  if (T > 64) return gemm_bf16_pipe_activated(s, x, w, act, out, T, N, K);
+  if (T > 64) return gemm_bf16_pipe_joined(s, x, w, bias, act, out, out_stride, split, second, second_stride, T, N, K);
   FusedArgs a = {};
-  a.x = (const uint16_t*)x; a.w = (const uint16_t*)w; a.out = out; a.act = act;
+  a.x = (const uint16_t*)x; a.w = (const uint16_t*)w; a.bias = bias; a.out = out; a.act = act;
+  a.second = (uint16_t*)second; a.split = split; a.out_stride = out_stride; a.second_stride = second_stride;
   a.T = T; a.N = N; a.K = K;
   a.k_per_split = (K + 63) / 64 * 64;
   return fused_norm<kEpiStore>(s, a, false, (N + 31) / 32, 1);

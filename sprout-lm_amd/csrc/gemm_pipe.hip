@@ -105,11 +105,16 @@ int gemm_bf16_pipe(hipStream_t s, const void* a, const void* w, int bias_dtype, 
   return pipe_shape<float>(s, a, w, bias, mode, out, T, N, K);
 }
 
-// The same with what StoreAct does to every number before it is stored (bfloat16, no bias).
-int gemm_bf16_pipe_activated(hipStream_t s, const void* a, const void* w, int act, void* out, int T, int N, int K) {
+// Two products of the same input in one: see sp_gemm_joined.
+int gemm_bf16_pipe_joined(hipStream_t s, const void* a, const void* w, const float* bias, int act, void* out, long long out_stride,
+                          int split, void* second, long long second_stride, int T, int N, int K) {
   RopeArgs epilogue = {};
   epilogue.act = act;
-  return pipe_shape<float>(s, a, w, nullptr, kStore, out, T, N, K, epilogue);
+  epilogue.second = (uint16_t*)second;
+  epilogue.split = split;
+  epilogue.out_stride = out_stride;
+  epilogue.second_stride = second_stride;
+  return pipe_shape<float>(s, a, w, bias, kStore, out, T, N, K, epilogue);
 }
 
 }  // namespace sprout

@@ -26,7 +26,8 @@ struct MlstmArgs {
   const int32_t *q_start, *q_len, *state_slots;
   float* memory;               // [slots, heads, vdim + 1, dim]
   float* maxima;               // [slots, heads]
-  void* out;                   // [T, heads * vdim]
+  void* out;                   // rows of out_stride numbers, the first heads * vdim of a row
+  long long out_stride;
 };
 
 __device__ __forceinline__ float log_input_gate(float x, float bias, float cap) { return cap * tanhf((x + bias) / cap); }
@@ -111,7 +112,7 @@ __global__ __launch_bounds__(1024) void mlstm_step_kernel(MlstmArgs a, int lanes
     }
     squares = block_sum(squares, scratch);      // (its barriers also publish o_row)
     const float unit = 1.0f / sqrtf(squares / float(V) + a.eps);
-    T* dst = out + (size_t(t) * a.heads + h) * V;
+    T* dst = out + size_t(t) * a.out_stride + h * V;
     if (v0 < V) dst[v0] = from_float<T>(((o_row[v0] * unit) * weight0) * sigmoid(gate0));
     for (int v = v0 + threads; v < V; v += threads)
       dst[v] = from_float<T>(((o_row[v] * unit) * a.norm[h * V + v]) * sigmoid(to_float(row[a.gate_off + h * V + v])));
@@ -200,7 +201,7 @@ __global__ __launch_bounds__(1024) void mlstm_stream_kernel(MlstmArgs a, int lan
     squares = block_sum(squares, scratch);      // (its barriers also publish o_row)
     const float unit = 1.0f / sqrtf(squares / float(V) + a.eps);
     for (int v = threadIdx.x; v < V; v += threads)
-      out[(size_t(t) * a.heads + h) * V + v] =
+      out[size_t(t) * a.out_stride + h * V + v] =
           from_float<T>(((o_row[v] * unit) * a.norm[h * V + v]) * sigmoid(to_float(row[a.gate_off + h * V + v])));
   }
   if (in && group == 0) *reinterpret_cast<float4*>(kept + size_t(V) * D) = norm;
@@ -248,7 +249,7 @@ __global__ __launch_bounds__(256) void mlstm_general_kernel(MlstmArgs a) {
     for (int v = threadIdx.x; v < V; v += 256) { const float x = os[v] * share; squares = fmaf(x, x, squares); }
     const float unit = 1.0f / sqrtf(block_sum(squares, scratch) / float(V) + a.eps);
     for (int v = threadIdx.x; v < V; v += 256)
-      out[(size_t(t) * a.heads + h) * V + v] =
+      out[size_t(t) * a.out_stride + h * V + v] =
           from_float<T>((((os[v] * share) * unit) * a.norm[h * V + v]) * sigmoid(to_float(row[a.gate_off + h * V + v])));
     __syncthreads();
   }
@@ -600,7 +601,7 @@ __global__ __launch_bounds__(64 * WAVES) void mlstm_chunk_apply_kernel(MlstmArgs
       for (int r = 0; r < 16; ++r) {
         const int i = 32 * ti + 8 * (r / 4) + 4 * hi + r % 4;
         if (i >= len) continue;
-        out[(size_t(first + i) * a.heads + h) * V + v] = from_float<bf16_t>(((o[t][ti][r] * unit[i]) * w) * sigmoid(gate[r]));
+        out[size_t(first + i) * a.out_stride + h * V + v] = from_float<bf16_t>(((o[t][ti][r] * unit[i]) * w) * sigmoid(gate[r]));
       }
     }
   }
@@ -686,7 +687,7 @@ extern "C" long long sp_mlstm_scratch_floats(int dtype, int heads, int dim, int 
 extern "C" int sp_mlstm(void* stream, int dtype, const void* proj, long long stride, int q_off, int k_off, int v_off, int gate_off,
                         int i_off, int f_off, int heads, int dim, int vdim, float cap, const float* bias_i, const float* bias_f,
                         const float* norm, float eps, const int32_t* q_start, const int32_t* q_len, const int32_t* state_slots,
-                        float* memory, float* maxima, void* out, int T, int n_seqs, int max_q_len, float* scratch) {
+                        float* memory, float* maxima, void* out, long long out_stride, int T, int n_seqs, int max_q_len, float* scratch) {
   SP_REQUIRE(heads > 0 && sp_mlstm_takes(dim, vdim), "sp_mlstm: no kernel for heads of %d and %d numbers", dim, vdim);
   SP_REQUIRE(cap > 0.f, "sp_mlstm: the gates' cap must be positive, not %g", double(cap));
   const long long qk = (long long)heads * dim, vg = (long long)heads * vdim;
@@ -694,12 +695,13 @@ extern "C" int sp_mlstm(void* stream, int dtype, const void* proj, long long str
                  stride >= q_off + qk && stride >= k_off + qk && stride >= v_off + vg && stride >= gate_off + vg &&
                  stride >= i_off + heads && stride >= f_off + heads,
              "sp_mlstm: rows of %lld numbers do not hold q, k, v and the gates", stride);
+  SP_REQUIRE(out_stride >= vg, "sp_mlstm: a row of %lld results does not hold the heads' outputs", out_stride);
   SP_REQUIRE(proj && bias_i && bias_f && norm && q_start && q_len && state_slots && memory && maxima && out, "sp_mlstm: null operand");
   SP_REQUIRE(dtype == kF32 || dtype == kBF16, "sp_mlstm: unsupported dtype %d", dtype);
   SP_REQUIRE(heads <= 65535, "sp_mlstm: %d heads are more than a launch's second dimension holds", heads);
   if (T == 0 || n_seqs == 0) return 0;
   const MlstmArgs a = {proj, stride, q_off, k_off, v_off, gate_off, i_off, f_off, heads, dim, vdim, cap, bias_i, bias_f, norm, eps,
-                       q_start, q_len, state_slots, memory, maxima, out};
+                       q_start, q_len, state_slots, memory, maxima, out, out_stride};
   hipStream_t s = (hipStream_t)stream;
   // whether rows of q, k and v (and the memory's) start at whole pieces of `numbers` numbers
   auto rows_at = [&](int numbers) {

@@ -278,12 +278,13 @@ __global__ __launch_bounds__(256) void qkv_prepare_kernel(PrepareArgs a) {
   }
 }
 
-// The difference of two maps' outputs, normed: out[t, h, :V] = (o / sqrt(mean(o^2) + eps)) * factor with
+// The difference of two maps' outputs, normed: out[t * stride + h * V + d] = (o / sqrt(mean(o^2) + eps)) * factor with
 // o = maps[t, 2 h] - lambda * maps[t, 2 h + 1], each map V of `width` numbers.  A wave per (token, head), its numbers in
 // registers (PER a lane) between the sum of squares and the store.
 template <typename TI, typename T, int PER>
 __global__ __launch_bounds__(256) void map_difference_kernel(const TI* __restrict__ maps, const float* __restrict__ lambda,
-                                                             float eps, float factor, T* __restrict__ out, int rows, int V, int width) {
+                                                             float eps, float factor, T* __restrict__ out, long long stride, int heads,
+                                                             int rows, int V, int width) {
   const int row = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   if (row >= rows) return;
   const float lam = *lambda;
@@ -296,10 +297,11 @@ __global__ __launch_bounds__(256) void map_difference_kernel(const TI* __restric
     sq = fmaf(o[i], o[i], sq);
   }
   const float unit = factor / sqrtf(wave_sum(sq) / float(V) + eps);
+  T* dst = out + size_t(row / heads) * stride + size_t(row % heads) * V;
 #pragma unroll
   for (int i = 0; i < PER; ++i) {
     const int d = lane + 64 * i;
-    if (d < V) out[size_t(row) * V + d] = from_float<T>(o[i] * unit);
+    if (d < V) dst[d] = from_float<T>(o[i] * unit);
   }
 }
 
@@ -308,13 +310,13 @@ __global__ __launch_bounds__(256) void map_difference_kernel(const TI* __restric
 using namespace sprout;
 
 extern "C" int sp_map_difference(void* stream, int in_dtype, const void* maps, int width, const float* lambda, float eps,
-                                 float factor, int dtype, void* out, int T, int heads, int vdim) {
-  SP_REQUIRE(T >= 0 && heads > 0 && vdim > 0 && vdim <= 512 && width >= vdim && maps && lambda && out, "sp_map_difference: bad arguments");
+                                 float factor, int dtype, void* out, long long out_stride, int T, int heads, int vdim) {
+  SP_REQUIRE(T >= 0 && heads > 0 && vdim > 0 && vdim <= 512 && width >= vdim && out_stride >= (long long)heads * vdim && maps && lambda && out, "sp_map_difference: bad arguments");
   SP_REQUIRE((in_dtype == kF32 || in_dtype == kBF16) && (dtype == kF32 || dtype == kBF16), "sp_map_difference: unsupported dtypes");
   if (T == 0) return 0;
   const int rows = T * heads;
   hipStream_t s = (hipStream_t)stream;
-#define SP_DIFF(TI, TT, PER) map_difference_kernel<TI, TT, PER><<<(rows + 3) / 4, 256, 0, s>>>((const TI*)maps, lambda, eps, factor, (TT*)out, rows, vdim, width)
+#define SP_DIFF(TI, TT, PER) map_difference_kernel<TI, TT, PER><<<(rows + 3) / 4, 256, 0, s>>>((const TI*)maps, lambda, eps, factor, (TT*)out, out_stride, heads, rows, vdim, width)
 #define SP_DIFF_TYPES(PER)                                                       \
   do {                                                                           \
     if (in_dtype == kF32 && dtype == kF32) SP_DIFF(float, float, PER);           \

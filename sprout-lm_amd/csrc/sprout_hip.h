@@ -45,9 +45,12 @@ int sp_pipe_plan(int kind, int T, int N, int K, int hd, int* plan);
 int sp_pipe_tiles(int tiles_t, int tiles_n, int* tile_of, int room);
 int sp_gemm_decode(void* stream, const void* x, const float* residual, int norm_w_dtype, const void* norm_w, float eps,
                    const void* w, int bias_dtype, const void* bias, int mode, void* out, int T, int N, int K);
-// out [T, N] (bfloat16) = act(x . w^T) with the activation in the product's epilogue, act 1 = max(v, 0)^2; bfloat16 operands.
-int sp_gemm_activated_takes(int T, int N, int K);
-int sp_gemm_activated(void* stream, const void* x, const void* w, int act, void* out, int T, int N, int K);
+// Two products of the same input in one (bfloat16 operands and results): with y = x . w^T + bias (float32 [N], may be null),
+// out[t * out_stride + n] = y[t, n] for n < split, second[t * second_stride + n - split] = act(y[t, n]) for the others; act 0 =
+// as it is, 1 = max(y, 0)^2.  split (0: all rows are the second product's), N and strides in fours.
+int sp_gemm_joined_takes(int T, int N, int K);
+int sp_gemm_joined(void* stream, const void* x, const void* w, const float* bias, int act, void* out, long long out_stride,
+                   int split, void* second, long long second_stride, int T, int N, int K);
 // q, k, v projection (+ bias), rotation of q and k, q to q_out [T, nq * hd], k and v into the paged pools.
 // With more than 64 tokens (head sizes that are multiples of 64) the tiled product does it in its epilogue;
 // cos_sin (may be null): the table of sp_rope_table for these positions, which saves it the sines and cosines.
@@ -155,9 +158,10 @@ int sp_qkv_prepare(void* stream, int dtype, const void* proj, long long stride, 
 // dim numbers of keys), while query row n (of nq, a multiple of maps) is map n % maps of its head: its numbers stand in q_out
 // where that map's do in a key, zeros elsewhere, so that its product with a whole key is the map's own.
 // out[t, h, :vdim] = o / sqrt(mean(o^2) + eps) * factor with o = maps[t, 2 h] - *lambda * maps[t, 2 h + 1]; maps [T, 2 heads,
-// width] of in_dtype (vdim numbers each, vdim up to 512), lambda one float on the device, out [T, heads * vdim] of dtype.
+// width] of in_dtype (vdim numbers each, vdim up to 512), lambda one float on the device, out of dtype, rows of out_stride
+// numbers (the first heads * vdim are written).
 int sp_map_difference(void* stream, int in_dtype, const void* maps, int width, const float* lambda, float eps, float factor,
-                      int dtype, void* out, int T, int heads, int vdim);
+                      int dtype, void* out, long long out_stride, int T, int heads, int vdim);
 
 // dst (dst_dtype) = src (src_dtype), n elements
 
@@ -340,14 +344,15 @@ long long sp_delta_scratch_floats(int heads, int dim, int vdim, int n_seqs, int 
 // (heads * vdim each) and two numbers per head (i, f) at their offsets.  Per head: i = cap tanh((i + bias_i) / cap), f =
 // logsigmoid(cap tanh((f + bias_f) / cap)); with a running maximum m, which starts at 0: m' = max(f + m, i), S <- exp(f + m - m') S
 // + exp(i - m') v k^T, n <- exp(f + m - m') n + exp(i - m') k, and with q' = dim^(-1/2) q: o = S q' / (max(|n . q'|, exp(-m')) + 1e-6).
-// out [T, heads * vdim] = o / sqrt(mean over vdim of o^2 + eps) * norm[heads * vdim] * sigmoid(gate).  memory float32
+// out (rows of out_stride numbers, the first heads * vdim of them) = o / sqrt(mean over vdim of o^2 + eps) * norm[heads * vdim] *
+// sigmoid(gate).  memory float32
 // [slots, heads, vdim + 1, dim]: S a row per value number, n as the last row; maxima float32 [slots, heads].  norm, biases
 // float32.
 int sp_mlstm_takes(int dim, int vdim);
 int sp_mlstm(void* stream, int dtype, const void* proj, long long stride, int q_off, int k_off, int v_off, int gate_off, int i_off,
              int f_off, int heads, int dim, int vdim, float cap, const float* bias_i, const float* bias_f, const float* norm,
              float eps, const int32_t* q_start, const int32_t* q_len, const int32_t* state_slots, float* memory, float* maxima,
-             void* out, int T, int n_seqs, int max_q_len, float* scratch);
+             void* out, long long out_stride, int T, int n_seqs, int max_q_len, float* scratch);
 // max_q_len, scratch: as for sp_retention, with sp_mlstm_scratch_floats numbers.
 long long sp_mlstm_scratch_floats(int dtype, int heads, int dim, int vdim, int n_seqs, int max_q_len, int T);
 

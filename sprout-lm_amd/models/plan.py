@@ -215,6 +215,8 @@ class ModelParts:
                     again[name] = mine[local]
             part.bind(mine)
             part.prepare(device, dtype)
+        for block in self.blocks:
+            block.join(dtype)
         if getattr(self.head, "tied", False):
             self.head.tie(self.embedding.w["weight"])
 

@@ -542,14 +542,14 @@ def qkv_prepare(proj: torch.Tensor, nq: int, nkv: int, dim: int, vdim: int, widt
 def map_difference(maps: torch.Tensor, width: int, factor: torch.Tensor, eps: float, scale: float, out: torch.Tensor, heads: int,
                    vdim: int) -> None:
     """out[t, h] = rms(maps[t, 2 h] - factor * maps[t, 2 h + 1]) * scale over vdim of `width` numbers a map (`eps` inside the
-    root); `factor`: one float32 number on the device."""
+    root), in the first heads * vdim columns of `out`; `factor`: one float32 number on the device."""
     _gpu(maps, "attention maps"); _gpu(out, "map difference"); _gpu(factor, "map factor")
     T = out.shape[0]
-    if maps.shape[0] < T or maps.shape[1] != 2 * heads * width or tuple(out.shape) != (T, heads * vdim) or not out.is_contiguous() \
+    if maps.shape[0] < T or maps.shape[1] != 2 * heads * width or out.shape[1] < heads * vdim or not out.is_contiguous() \
             or not maps.is_contiguous() or factor.dtype != torch.float32 or factor.numel() != 1:
         raise KernelError(f"map_difference: maps {tuple(maps.shape)}, factor and result {tuple(out.shape)} do not fit")
     check(library().sp_map_difference(_stream(), _code(maps, "attention maps"), maps.data_ptr(), width, factor.data_ptr(),
-                                      float(eps), float(scale), _code(out, "map difference"), out.data_ptr(), T, heads, vdim))
+                                      float(eps), float(scale), _code(out, "map difference"), out.data_ptr(), out.shape[1], T, heads, vdim))
 
 
 STORE, ACCUMULATE, STORE_F32 = 0, 1, 2
@@ -1036,19 +1036,44 @@ def activation(x: torch.Tensor, kind: str) -> None:
 FOLDED_ACTIVATIONS = {"relu_squared": 1}      # unary activations that the plain product has in its epilogue
 
 
+def joined_takes(T: int, N: int, K: int) -> bool:
+    """Whether `gemm_joined` takes T x N x K."""
+    return K % 8 == 0 and bool(library().sp_gemm_joined_takes(int(T), int(N), int(K)))
+
+
+def gemm_joined(x: torch.Tensor, w: torch.Tensor, bias, out, split: int, second: torch.Tensor, column: int, kind: str) -> None:
+    """Two products of the same input in one kernel (bfloat16): with y = x . w^T + bias (float32 [N] or None), out [T, split] =
+    the first `split` columns of y, and columns `column` .. of the rows of `second` = act of the others (`kind`: one of
+    FOLDED_ACTIVATIONS).  split 0: no `out`."""
+    _gpu(x, "input"); _gpu(w, "weight"); _gpu(second, "second output")
+    T, (N, K) = x.shape[0], w.shape
+    act = variant_code(FOLDED_ACTIVATIONS, kind, "activation")
+    if x.dtype != torch.bfloat16 or w.dtype != torch.bfloat16 or second.dtype != torch.bfloat16 or x.shape[1] != K \
+            or not (x.is_contiguous() and w.is_contiguous() and second.is_contiguous()):
+        raise KernelError("gemm_joined: bfloat16 operands without gaps expected")
+    if second.shape[0] != T or column < 0 or column + N - split > second.shape[1]:
+        raise KernelError(f"gemm_joined: {N - split} columns do not fit rows of {second.shape[1]} from {column} on")
+    if split:
+        _gpu(out, "first output")
+        if out.dtype != torch.bfloat16 or tuple(out.shape) != (T, split) or not out.is_contiguous():
+            raise KernelError(f"gemm_joined: the first output must be bfloat16 [{T}, {split}], got {tuple(out.shape)} {out.dtype}")
+    if bias is not None:
+        _gpu(bias, "bias")
+        if bias.dtype != torch.float32 or bias.numel() != N:
+            raise KernelError(f"gemm_joined: the bias must hold {N} float32 values")
+    check(library().sp_gemm_joined(_stream(), x.data_ptr(), w.data_ptr(), _ptr(bias), act, out.data_ptr() if split else None, split, split,
+                                   second.data_ptr() + 2 * column, second.shape[1], T, N, K))
+
+
 def gemm_activated(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, kind: str) -> bool:
     """out = act(x . w^T) in one kernel (bfloat16, no bias).  Returns False (and does nothing) where no product kernel has the
     activation in its epilogue for the call; the caller then multiplies and activates in turn."""
-    act = FOLDED_ACTIVATIONS.get(kind)
-    if act is None or x.dtype != torch.bfloat16 or w.dtype != torch.bfloat16 or out.dtype != torch.bfloat16:
+    if kind not in FOLDED_ACTIVATIONS or x.dtype != torch.bfloat16 or w.dtype != torch.bfloat16 or out.dtype != torch.bfloat16:
         return False
     T, (N, K) = x.shape[0], w.shape
-    if x.shape[1] != K or tuple(out.shape) != (T, N) or not (x.is_contiguous() and w.is_contiguous() and out.is_contiguous()):
-        raise KernelError(f"gemm_activated: shapes do not fit: x {tuple(x.shape)}, w {tuple(w.shape)}, out {tuple(out.shape)}")
-    if T == 0 or K % 8 or (x.data_ptr() | w.data_ptr()) & 15 or not library().sp_gemm_activated_takes(T, N, K):
+    if T == 0 or N % 4 or (x.data_ptr() | w.data_ptr()) & 15 or not joined_takes(T, N, K):
         return False
-    _gpu(x, "input"); _gpu(w, "weight"); _gpu(out, "output")
-    check(library().sp_gemm_activated(_stream(), x.data_ptr(), w.data_ptr(), act, out.data_ptr(), T, N, K))
+    gemm_joined(x, w, None, None, 0, out, 0, kind)
     return True
 
 
@@ -1209,10 +1234,11 @@ def mlstm(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, gate_off: int,
           vdim: int, cap: float, bias_i: torch.Tensor, bias_f: torch.Tensor, norm: torch.Tensor, eps: float, q_start, q_len,
           state_slots, n_seqs: int, memory: torch.Tensor, maxima: torch.Tensor, out: torch.Tensor, max_q_len: int = 0,
           workspace=None) -> None:
-    """The matrix memory of sp_mlstm (sprout_hip.h) on a step's tokens.  `max_q_len`, `workspace`: as for `rglru`."""
+    """The matrix memory of sp_mlstm (sprout_hip.h) on a step's tokens, its outputs in the first heads * vdim columns of `out`.
+    `max_q_len`, `workspace`: as for `rglru`."""
     T = out.shape[0]
     _gpu(proj, "projections"); _gpu(out, "memory output"); _gpu(memory, "memory"); _gpu(maxima, "running maxima")
-    if proj.shape[0] < T or out.dtype != proj.dtype or tuple(out.shape) != (T, heads * vdim) or not out.is_contiguous():
+    if proj.shape[0] < T or out.dtype != proj.dtype or out.shape[1] < heads * vdim or not out.is_contiguous():
         raise KernelError(f"mlstm: projections {tuple(proj.shape)} {proj.dtype} and output {tuple(out.shape)} {out.dtype} do not fit")
     if max(q_off, k_off) + heads * dim > proj.shape[1] or max(v_off, gate_off) + heads * vdim > proj.shape[1] \
             or max(i_off, f_off) + heads > proj.shape[1] or min(q_off, k_off, v_off, gate_off, i_off, f_off) < 0:
@@ -1232,7 +1258,7 @@ def mlstm(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, gate_off: int,
     check(library().sp_mlstm(_stream(), code, proj.data_ptr(), proj.shape[1], q_off, k_off, v_off, gate_off, i_off, f_off, heads,
                              dim, vdim, float(cap), bias_i.data_ptr(), bias_f.data_ptr(), norm.data_ptr(), float(eps),
                              q_start.data_ptr(), q_len.data_ptr(), state_slots.data_ptr(), memory.data_ptr(), maxima.data_ptr(),
-                             out.data_ptr(), T, n_seqs, int(max_q_len) if scratch is not None else 0, _ptr(scratch)))
+                             out.data_ptr(), out.shape[1], T, n_seqs, int(max_q_len) if scratch is not None else 0, _ptr(scratch)))
 
 
 def gemm_from_residual(residual: torch.Tensor, norm_weight: torch.Tensor, eps: float, w: torch.Tensor, out: torch.Tensor,

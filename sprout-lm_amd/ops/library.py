@@ -36,8 +36,8 @@ def _declare(lib):
         "sp_pipe_tiles": [c_int, c_int, ctypes.POINTER(c_int), c_int],
         "sp_gemm_decode": [c_void, c_void, c_void, c_int, c_void, c_float, c_void, c_int, c_void, c_int, c_void, c_int,
                            c_int, c_int],
-        "sp_gemm_activated_takes": [c_int] * 3,
-        "sp_gemm_activated": [c_void, c_void, c_void, c_int, c_void, c_int, c_int, c_int],
+        "sp_gemm_joined_takes": [c_int] * 3,
+        "sp_gemm_joined": [c_void, c_void, c_void, c_void, c_int, c_void, c_i64, c_int, c_void, c_i64, c_int, c_int, c_int],
         "sp_qkv_rope_cache": [c_void, c_void, c_void, c_int, c_void, c_float, c_void, c_int, c_void, c_void, c_void,
                               c_void, c_int, c_void, c_void, c_void, c_int, c_int, c_int, c_int, c_int, c_int, c_void, c_int],
         "sp_rope_table": [c_void, c_void, c_void, c_void, c_int, c_float, c_void, c_int],
@@ -87,10 +87,10 @@ def _declare(lib):
         "sp_qkv_prepare": [c_void, c_int, c_void, c_i64, c_int, c_int, c_int, c_int, c_int, c_void, c_void, c_float, c_void,
                            c_void, c_void, c_int, c_void, c_void, c_int, c_void, c_void, c_void, c_int, c_int, c_void, c_int,
                            c_float, c_int, c_void, c_int],
-        "sp_map_difference": [c_void, c_int, c_void, c_int, c_void, c_float, c_float, c_int, c_void, c_int, c_int, c_int],
+        "sp_map_difference": [c_void, c_int, c_void, c_int, c_void, c_float, c_float, c_int, c_void, c_i64, c_int, c_int, c_int],
         "sp_mlstm_takes": [c_int] * 2,
         "sp_mlstm": [c_void, c_int, c_void, c_i64, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_void,
-                     c_void, c_void, c_float, c_void, c_void, c_void, c_void, c_void, c_void, c_int, c_int, c_int, c_void],
+                     c_void, c_void, c_float, c_void, c_void, c_void, c_void, c_void, c_void, c_i64, c_int, c_int, c_int, c_void],
         "sp_expert_down": [c_void, c_int, c_void, c_void, c_void, c_void, c_int, c_int, c_void, c_int, c_int, c_int, c_int],
         "sp_route_combine": [c_void, c_void, c_void, c_void, c_int, c_void, c_int, c_int],
         "sp_route_sigmoid": [c_void, c_void, c_void, c_void, c_int, c_int, c_int, c_int, c_void, c_void, c_void, c_void],

@@ -153,10 +153,37 @@ class Mixer(Part):
         """target (float32) += the mixer's output, or target = it with `accumulate` False."""
         raise NotImplementedError
 
+    # For a mixer that is one product of its input, a middle, and one product into the residual (`joins`): a parallel block
+    # whose feed-forward is of that kind too makes one product of the two first ones and one of the two last ones.
+    # `give_matrices` hands over (first matrix, its bias or None, last matrix), and `forward_middle` brings the first
+    # product's rows `proj` to what enters the last one, in the first `middle_width` columns of the rows of `out`.
+    middle_width = 0
+
+    def joins(self) -> bool:
+        return False
+
+    def first_rows(self) -> int:
+        """Rows of the first matrix."""
+        raise NotImplementedError
+
+    def give_matrices(self):
+        raise NotImplementedError
+
+    def forward_middle(self, ctx, proj, cache, out) -> None:
+        raise NotImplementedError
+
 
 class FeedForward(Part):
     def forward(self, ctx, h, residual):
         """residual += feed_forward(h), token by token."""
+        raise NotImplementedError
+
+    # As Mixer.joins: the feed-forward is down(act(up(h))) with `activation` one that the products have in their epilogues;
+    # `give_matrices` hands over (up, down).
+    def joins(self) -> bool:
+        return False
+
+    def give_matrices(self):
         raise NotImplementedError
 
     def forward_from_residual(self, ctx, norm, residual) -> bool:
@@ -189,6 +216,9 @@ class Block(Part):
         """The block's parts by the names under which the model plan gave them; everything the engine wants of a
         block's parts (tensors, cache needs, costs, whether they may be recorded) it asks through this."""
         raise NotImplementedError
+
+    def join(self, dtype) -> None:
+        """Called once, after the block's parts have received their tensors: the place to make one matrix of several parts'."""
 
     def forward(self, ctx, residual, caches: dict):
         """Run the block on the step's tokens.  `caches`: part name -> what that part's `cache_spec` asked for in

@@ -1,6 +1,9 @@
 """Arrangement of parts in a layer (reference: src/qwen.ts:164-202)."""
 from __future__ import annotations
 
+import torch
+
+from .. import ops
 from .base import Block, register_part
 
 
@@ -48,7 +51,9 @@ class PreNormBlock(Block):
 class ParallelBlock(Block):
     """x += mixer(norm_a(x)) + feed_forward(norm_b(x)): both norms read the same x, so both are taken before
     either part adds into the float32 residual stream.  `ffn` (and its norm) may be absent.  A feed-forward without a
-    norm of its own (`ffn_norm` None) reads norm_a(x), the mixer's input."""
+    norm of its own (`ffn_norm` None) reads norm_a(x), the mixer's input: where both sublayers can (`Mixer.joins`,
+    `FeedForward.joins`, bfloat16), their first products are then one product, whose feed-forward columns leave it activated,
+    and their last products one product over both sublayers' rows side by side."""
 
     graph_safe = True
 
@@ -56,6 +61,34 @@ class ParallelBlock(Block):
 
     def __init__(self, mixer_norm, mixer, ffn_norm=None, ffn=None):
         self.mixer_norm, self.mixer, self.ffn_norm, self.ffn = mixer_norm, mixer, ffn_norm, ffn
+        self.w_first = None
+
+    def join(self, dtype):
+        if (dtype != torch.bfloat16 or self.ffn is None or self.ffn_norm is not None or not self.mixer.joins() or not self.ffn.joins()
+                or self.mixer.middle_width % 8 or self.ffn.inner % 8):
+            return
+        rows, width = self.mixer.first_rows() + self.ffn.inner, self.ffn.hidden
+        if self.mixer.first_rows() % 8 or width % 64 or not ops.joined_takes(1, rows, width) or not ops.joined_takes(65, rows, width):
+            return
+        first, bias, last = self.mixer.give_matrices()
+        up, down = self.ffn.give_matrices()
+        self.w_first = torch.cat([first, up], dim=0).contiguous()
+        self.w_last = torch.cat([last, down], dim=1).contiguous()
+        self.split, self.b_first = first.shape[0], None
+        if bias is not None:
+            self.b_first = torch.cat([bias.to(torch.float32), torch.zeros(up.shape[0], device=bias.device)]).contiguous()
+
+    def _forward_joined(self, ctx, h, residual, cache):
+        T = h.shape[0]
+        proj = ctx.buffer("parallel_first", (T, self.split), ctx.act_dtype)
+        middle = ctx.buffer("parallel_middle", (T, self.w_last.shape[1]), ctx.act_dtype)
+        if T <= 64:      # few tokens: a launch less
+            ops.gemm_joined(h, self.w_first, self.b_first, proj, self.split, middle, self.mixer.middle_width, self.ffn.activation)
+        else:      # (many: the two shapes each find tiles that fit them better than their sum does)
+            ops.gemm(h, self.w_first[:self.split], proj, bias=None if self.b_first is None else self.b_first[:self.split])
+            ops.gemm_joined(h, self.w_first[self.split:], None, None, 0, middle, self.mixer.middle_width, self.ffn.activation)
+        self.mixer.forward_middle(ctx, proj, cache, middle)
+        ops.gemm(middle, self.w_last, residual, accumulate=True)
 
     def parts(self):
         named = {"mixer_norm": self.mixer_norm, "mixer": self.mixer}
@@ -76,6 +109,9 @@ class ParallelBlock(Block):
             if pair is None or not pair(ctx, self.ffn_norm, residual, h, h2):
                 self.mixer_norm.forward(ctx, residual, h)
                 self.ffn_norm.forward(ctx, residual, h2)
+        if self.w_first is not None:
+            self._forward_joined(ctx, h, residual, caches.get("mixer"))
+            return
         self.mixer.forward(ctx, h, residual, caches.get("mixer"))
         if self.ffn is not None:
             self.ffn.forward(ctx, h2, residual)
@@ -101,7 +137,6 @@ class ScaledParallelBlock(Block):
         return named
 
     def forward(self, ctx, residual, caches):
-        import torch
         T, H = residual.shape
         h = ctx.buffer("normed", (T, H), ctx.act_dtype)
         self.mixer_norm.forward(ctx, residual, h)

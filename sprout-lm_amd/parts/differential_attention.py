@@ -52,6 +52,7 @@ class DifferentialAttention(Mixer):
         self.scale, self.diff, self.eps, self.position = float(scale), float(diff), float(eps), position
         self.qkv_bias, self.window, self.page_tokens = bool(qkv_bias), window, page_tokens
         self.names = tuple(tensors)
+        self.middle_width = heads * vdim
 
     # ------------------------------------------------------------------ what it keeps and costs
     def cache_spec(self):
@@ -92,10 +93,26 @@ class DifferentialAttention(Mixer):
         return [self.position]
 
     # ------------------------------------------------------------------ the step
+    def joins(self):
+        return True
+
+    def first_rows(self):
+        return self.w_qkv.shape[0]
+
+    def give_matrices(self):
+        given, self.w_qkv, self.w_o = (self.w_qkv, self.b_qkv, self.w_o), None, None
+        return given
+
     def forward(self, ctx, h, residual, cache):
-        T, H, G, W = h.shape[0], self.heads, self.kv_heads, self.width
+        T = h.shape[0]
         proj = ctx.buffer("qkv", (T, self.w_qkv.shape[0]), ctx.act_dtype)
         ops.gemm(h, self.w_qkv, proj, bias=self.b_qkv)
+        mixed = ctx.buffer("map_difference", (T, self.middle_width), ctx.act_dtype)
+        self.forward_middle(ctx, proj, cache, mixed)
+        ops.gemm(mixed, self.w_o, residual, accumulate=True)
+
+    def forward_middle(self, ctx, proj, cache, out):
+        T, H, G, W = proj.shape[0], self.heads, self.kv_heads, self.width
         queries = ctx.buffer("padded_q", (T, 2 * H * W), ctx.act_dtype)
         writes = cache.writes
         rotary = getattr(self.position, "rotary_dim", 0)
@@ -108,6 +125,4 @@ class DifferentialAttention(Mixer):
         maps = ctx.buffer("attn", (T, 2 * H * W), ctx.act_dtype)
         ops.attention(queries, 2 * H * W, cache.k, cache.v, cache.block_tables, ctx.attention, maps, 2 * H, G, W, self.window,
                       self.scale, workspace=lambda n: ctx.buffer("attention_partials", (n,), torch.float32), kind=ctx.attention_kind)
-        mixed = ctx.buffer("map_difference", (T, H * self.vdim), ctx.act_dtype)
-        ops.map_difference(maps, W, self.factor, self.eps, 1.0 - self.diff, mixed, H, self.vdim)
-        ops.gemm(mixed, self.w_o, residual, accumulate=True)
+        ops.map_difference(maps, W, self.factor, self.eps, 1.0 - self.diff, out, H, self.vdim)

@@ -63,6 +63,7 @@ class LatentAttention(Mixer):
         self.page_tokens, self.q_rank, self.sinks = page_tokens, q_rank, bool(sinks)
         defaults = ("q", "dkv", "dkv.norm", "uk", "uv", "g", "o", "dq", "dq.norm", "uq", "sink")
         self.names = tuple(tensors) + defaults[len(tensors):]
+        self.middle_width = heads * vdim
 
     # ------------------------------------------------------------------ what it keeps and costs
     def cache_spec(self):
@@ -128,10 +129,26 @@ class LatentAttention(Mixer):
         return [self.position]
 
     # ------------------------------------------------------------------ the step
+    def joins(self):
+        return True
+
+    def first_rows(self):
+        return self.w_in.shape[0]
+
+    def give_matrices(self):
+        given, self.w_in, self.w_o = (self.w_in, None, self.w_o), None, None
+        return given
+
     def forward(self, ctx, h, residual, cache):
-        T, H, W = h.shape[0], self.heads, self.width
+        T = h.shape[0]
         proj = ctx.buffer("latent_proj", (T, self.w_in.shape[0]), ctx.act_dtype)
         ops.gemm(h, self.w_in, proj)
+        values = ctx.buffer("latent_values", (T, self.middle_width), ctx.act_dtype)
+        self.forward_middle(ctx, proj, cache, values)
+        ops.gemm(values, self.w_o, residual, accumulate=True)
+
+    def forward_middle(self, ctx, proj, cache, out):
+        T, H, W = proj.shape[0], self.heads, self.width
         queries = ctx.buffer("latent_q", (T, H * W), ctx.act_dtype)
         writes = cache.writes
         turn = (ctx.positions, self.position.freq, self.position.rotary_dim, self.position.magnitude, self.position.pairing)
@@ -152,7 +169,4 @@ class LatentAttention(Mixer):
         ops.attention(queries, H * W, cache.k, cache.v, cache.block_tables, ctx.attention, mixed, H, 1, W, self.window,
                       self.scale, workspace=lambda n: ctx.buffer("attention_partials", (n,), torch.float32),
                       kind=ctx.attention_kind, sinks=self.sink)
-        values = ctx.buffer("latent_values", (T, H * self.vdim), ctx.act_dtype)
-        ops.head_gemm(mixed, 0, W, self.w_uv, values, 0, self.vdim, gate=proj if self.gated else None,
-                      gate_offset=self.gate_off)
-        ops.gemm(values, self.w_o, residual, accumulate=True)
+        ops.head_gemm(mixed, 0, W, self.w_uv, out, 0, self.vdim, gate=proj if self.gated else None, gate_offset=self.gate_off)

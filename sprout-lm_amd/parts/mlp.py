@@ -128,6 +128,13 @@ class DenseMLP(FeedForward):
         self.b_down = tensors[down + self.bias] if self.bias is not None else None
         self.w = {}
 
+    def joins(self):
+        return self.bias is None and self.activation in ops.FOLDED_ACTIVATIONS
+
+    def give_matrices(self):
+        given, self.w_up, self.w_down = (self.w_up, self.w_down), None, None
+        return given
+
     def forward_from_residual(self, ctx, norm, residual) -> bool:
         """A decode step's few tokens: the norm as the prologue of the up product, a launch less."""
         fold = norm.fold()

@@ -36,6 +36,7 @@ class MatrixLSTM(Mixer):
             raise ConfigError(f"No kernel for a matrix memory with heads of {dim} and {vdim} numbers.")
         self.hidden, self.heads, self.dim, self.vdim, self.gate_cap, self.eps = hidden, heads, dim, vdim, float(gate_cap), float(eps)
         self.names = tuple(tensors)
+        self.middle_width = heads * vdim
 
     # ------------------------------------------------------------------ what it keeps and costs
     def cache_spec(self):
@@ -70,13 +71,27 @@ class MatrixLSTM(Mixer):
         self.w = {}
 
     # ------------------------------------------------------------------ the step
+    def joins(self):
+        return True
+
+    def first_rows(self):
+        return self.w_in.shape[0]
+
+    def give_matrices(self):
+        given, self.w_in, self.w_o = (self.w_in, None, self.w_o), None, None
+        return given
+
     def forward(self, ctx, h, residual, cache):
-        q, k, v, g, i, f, *_ = self.names
-        T, H, D, V = h.shape[0], self.heads, self.dim, self.vdim
+        T = h.shape[0]
         proj = ctx.buffer("mlstm_in", (T, self.w_in.shape[0]), ctx.act_dtype)
         ops.gemm(h, self.w_in, proj)
-        out = ctx.buffer("mlstm_out", (T, H * V), ctx.act_dtype)
-        ops.mlstm(proj, *(self.at[name] for name in (q, k, v, g, i, f)), H, D, V, self.gate_cap, self.b_i, self.b_f, self.w_norm,
-                  self.eps, ctx.q_start, ctx.q_len, ctx.state_slots, ctx.n_seqs, cache["memory"].state, cache["max"].state, out,
-                  max_q_len=ctx.max_q_len, workspace=lambda n: ctx.buffer("mlstm_chunks", (n,), torch.float32))
+        out = ctx.buffer("mlstm_out", (T, self.middle_width), ctx.act_dtype)
+        self.forward_middle(ctx, proj, cache, out)
         ops.gemm(out, self.w_o, residual, accumulate=True)
+
+    def forward_middle(self, ctx, proj, cache, out):
+        q, k, v, g, i, f, *_ = self.names
+        ops.mlstm(proj, *(self.at[name] for name in (q, k, v, g, i, f)), self.heads, self.dim, self.vdim, self.gate_cap, self.b_i,
+                  self.b_f, self.w_norm, self.eps, ctx.q_start, ctx.q_len, ctx.state_slots, ctx.n_seqs, cache["memory"].state,
+                  cache["max"].state, out, max_q_len=ctx.max_q_len,
+                  workspace=lambda n: ctx.buffer("mlstm_chunks", (n,), torch.float32))
