@@ -61,6 +61,64 @@ def test_square_of_relu_feed_forward(dtype, T, hidden, inner):
     close(residual.cpu().numpy(), V.dense_ff(w, "", x, store_of(dtype)), dtype, "feed-forward", f32=2e-5, bf16=1e-2)
 
 
+@pytest.mark.parametrize("T", [1, 16, 17, 64, 65, 300])
+@pytest.mark.parametrize("split,second,K,bias", [(0, 64, 64, False), (40, 96, 128, True), (136, 24, 192, False), (256, 260, 64, True)])
+def test_two_products_of_one_input(T, split, second, K, bias):
+    """Rows of one matrix that go to two tensors, the second activated and between other columns, for few and many tokens."""
+    from sprout_lm_amd import ops
+    rng = np.random.default_rng(T + split)
+    x, w = (rounded(rng.standard_normal(shape), torch.bfloat16) for shape in ((T, K), (split + second, K)))
+    b = rng.standard_normal(split + second).astype(np.float32) if bias else None
+    out = torch.full((T, max(split, 4)), 7.0, dtype=torch.bfloat16, device=DEV)
+    rows = torch.full((T, second + 12), 7.0, dtype=torch.bfloat16, device=DEV)
+    ops.gemm_joined(dev(x, torch.bfloat16), dev(w, torch.bfloat16), None if b is None else dev(b), out if split else None, split, rows, 8,
+                    "relu_squared")
+    y = x.astype(np.float64) @ w.astype(np.float64).T + (0.0 if b is None else b)
+    got = rows.float().cpu().numpy()
+    if split:
+        close(out.float().cpu().numpy(), y[:, :split], torch.bfloat16, "first product", bf16=2.0 ** -8)
+    close(got[:, 8:8 + second], np.maximum(y[:, split:], 0.0) ** 2, torch.bfloat16, "second product", bf16=2.0 ** -8)
+    assert np.all(got[:, :8] == 7.0) and np.all(got[:, 8 + second:] == 7.0)
+
+
+@pytest.mark.parametrize("page,window,keep,sinks", [(16, None, 0, True), (8, 100, 0, True), (16, 70, 5, False), (12, 100, 0, False), (32, None, 0, False)])
+@pytest.mark.parametrize("width", [160, 192, 256])
+def test_wide_heads(width, page, window, keep, sinks):
+    """Heads above 128 numbers in bfloat16: portions, single queries and long contexts beside each other, every number of heads
+    over a key head that changes how a block is cut, windows, kept first keys, sinks, pages of a power of two and not."""
+    from sprout_lm_amd import ops
+    from sprout_lm_amd.ops.kernels import AttentionBatch
+    rng = np.random.default_rng(width + page)
+    lens, ctx = [33, 1, 1, 5, 150, 1], [300, 400, 7, 1400, 150, 1]
+    T, table, pages = sum(lens), [], 0
+    order = rng.permutation(sum(-(-c // page) for c in ctx))
+    for c in ctx:
+        n = -(-c // page)
+        table.append(list(order[pages:pages + n]) + [0] * (-(-max(ctx) // page) - n))
+        pages += n
+    for nq, nkv in ((1, 1), (2, 1), (3, 1), (6, 1), (16, 1), (20, 1), (4, 2)):
+        q = rounded(rng.standard_normal((T, nq, width)), torch.bfloat16)
+        k, v = (rounded(rng.standard_normal((pages * page, nkv, width)), torch.bfloat16) for _ in range(2))
+        k_pool = dev(k.reshape(pages, page, nkv, width).transpose(0, 2, 1, 3), torch.bfloat16).contiguous()
+        v_pool = dev(v.reshape(pages, page, nkv, width).transpose(0, 2, 3, 1), torch.bfloat16).contiguous()
+        sink = rng.normal(2, 2, nq).astype(np.float32) if sinks else None
+        out = torch.full((T, nq * width), float("nan"), dtype=torch.bfloat16, device=DEV)
+        ops.attention(dev(q.reshape(T, -1), torch.bfloat16), nq * width, k_pool, v_pool, torch.tensor(table, dtype=torch.int32, device=DEV),
+                      AttentionBatch.build(lens, ctx, DEV), out, nq, nkv, width, window, 1.5 * width ** -0.5,
+                      sinks=None if sink is None else dev(sink), keep_first=keep)
+        got, first = out.float().cpu().numpy().reshape(T, nq, width), 0
+        for s, (n, c) in enumerate(zip(lens, ctx)):
+            slots = np.array([table[s][p // page] * page + p % page for p in range(c)])
+            pos, key = np.arange(c - n, c)[:, None], np.arange(c)[None, :]
+            mask = (key <= pos) & ((pos - key < (window or c)) | (key < keep))
+            for h in range(nq):
+                g = h // (nq // nkv)
+                score = q[first:first + n, h].astype(np.float64) @ k[slots, g].astype(np.float64).T * (1.5 * width ** -0.5)
+                want = V.softmax(score, mask, None if sink is None else float(sink[h])) @ v[slots, g].astype(np.float64)
+                close(got[first:first + n, h], want, torch.bfloat16, f"{nq} over {nkv}, request {s}, head {h}", bf16=1.5e-2)
+            first += n
+
+
 class Scratch:
     """What a part asks of a step that carries no sequences."""
 
