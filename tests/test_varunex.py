@@ -76,7 +76,7 @@ def test_sizes_that_are_refused():
                 make_part("mixer", kind, **dict(good, **bad))
 
 
-@pytest.mark.parametrize("dims,base,scaling", [(12, 50000.0, (4.0, 1.0, 4.0, 512.0)), (8, 100.0, (16.0, 0.5, 3.0, 60.0)), (6, 20.0, (2.0, 2.0, 2.0, 30.0)),
+@pytest.mark.parametrize("dims,base,scaling", [(10, 30000.0, (6.0, 1.0, 5.0, 400.0)), (8, 100.0, (16.0, 0.5, 3.0, 60.0)), (6, 20.0, (2.0, 2.0, 2.0, 30.0)),
                                                (16, 1e6, None)])
 def test_frequencies_blended_by_wavelength(dims, base, scaling):
     """The engine's table and the plain one, which decides by wavelength; short waves kept, long ones stretched."""

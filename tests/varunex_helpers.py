@@ -58,7 +58,7 @@ ODD = model(100, 77, [
 GENERAL = model(128, 300, [
     layer(latent(4, 16, 16, 32, 64, 48, 0.2, rot(16, 1000.0, (8.0, 1.0, 4.0, 64.0))), 96),
     layer(difference(4, 1, 16, 32, 0.3, 0.35, rot(8, 250.0), 24), 64),
-    layer(memory(4, 32, 64, 10.0), 64),
+    layer(memory(3, 32, 56, 10.0), 64),
     layer(difference(4, 2, 32, 64, 0.2, 0.5, rot(32, 5000.0, (4.0, 1.0, 4.0, 128.0)), 100), 80),
     layer(memory(2, 16, 40, 15.0), 48),
 ], eps=1e-6)
