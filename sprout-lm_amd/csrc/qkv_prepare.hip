@@ -311,7 +311,7 @@ using namespace sprout;
 
 extern "C" int sp_map_difference(void* stream, int in_dtype, const void* maps, int width, const float* lambda, float eps,
                                  float factor, int dtype, void* out, long long out_stride, int T, int heads, int vdim) {
-  SP_REQUIRE(T >= 0 && heads > 0 && vdim > 0 && vdim <= 512 && width >= vdim && out_stride >= (long long)heads * vdim && maps && lambda && out, "sp_map_difference: bad arguments");
+  SP_REQUIRE(T >= 0 && heads > 0 && vdim > 0 && vdim <= 640 && width >= vdim && out_stride >= (long long)heads * vdim && maps && lambda && out, "sp_map_difference: bad arguments");
   SP_REQUIRE((in_dtype == kF32 || in_dtype == kBF16) && (dtype == kF32 || dtype == kBF16), "sp_map_difference: unsupported dtypes");
   if (T == 0) return 0;
   const int rows = T * heads;
@@ -326,7 +326,7 @@ extern "C" int sp_map_difference(void* stream, int in_dtype, const void* maps, i
   } while (0)
   if (vdim <= 128) SP_DIFF_TYPES(2);
   else if (vdim <= 256) SP_DIFF_TYPES(4);
-  else SP_DIFF_TYPES(8);
+  else SP_DIFF_TYPES(10);
 #undef SP_DIFF_TYPES
 #undef SP_DIFF
   return check_launch("sp_map_difference");

@@ -158,7 +158,7 @@ int sp_qkv_prepare(void* stream, int dtype, const void* proj, long long stride, 
 // dim numbers of keys), while query row n (of nq, a multiple of maps) is map n % maps of its head: its numbers stand in q_out
 // where that map's do in a key, zeros elsewhere, so that its product with a whole key is the map's own.
 // out[t, h, :vdim] = o / sqrt(mean(o^2) + eps) * factor with o = maps[t, 2 h] - *lambda * maps[t, 2 h + 1]; maps [T, 2 heads,
-// width] of in_dtype (vdim numbers each, vdim up to 512), lambda one float on the device, out of dtype, rows of out_stride
+// width] of in_dtype (vdim numbers each, vdim up to 640), lambda one float on the device, out of dtype, rows of out_stride
 // numbers (the first heads * vdim are written).
 int sp_map_difference(void* stream, int in_dtype, const void* maps, int width, const float* lambda, float eps, float factor,
                       int dtype, void* out, long long out_stride, int T, int heads, int vdim);

@@ -70,7 +70,7 @@ GATE_ACTIVATIONS = {"silu": 0,           # silu(g) * u
 HEAD_GATES = {"silu": 0, "sigmoid": 1}   # what a projection passes before it multiplies a head's normed read-out
 SCORE_STAGES = {"scaled_dot": 0,         # what stands between q . k and the softmax: the scale and nothing else,
                 "capped": 1}             # or the scaled product s squashed to cap * tanh(s / cap)
-MAX_HEAD_DIM = 512                       # the largest head size any attention kernel takes
+MAX_HEAD_DIM = 640                       # the largest head size any attention kernel takes
 
 
 def variant_code(table: dict, name: str, what: str) -> int:
@@ -83,7 +83,7 @@ def variant_code(table: dict, name: str, what: str) -> int:
 def check_attention_sizes(heads: int, kv_heads: int, head_dim: int) -> None:
     """Raises KernelError unless some attention kernel takes these sizes (any page size goes with them).
     Head sizes of 16 ... 96 in steps of 16, 128, 160, 192 and 256 run on the matrix cores in bfloat16, float32 in steps of 16 up
-    to 256 on the matrix cores' float32 instructions, every other size up to 512 on the general kernel."""
+    to 256 on the matrix cores' float32 instructions, every other size up to 640 on the general kernel."""
     if kv_heads <= 0 or heads <= 0 or heads % kv_heads:
         raise KernelError(f"attention: {heads} query heads do not divide into {kv_heads} key/value heads")
     if not 0 < head_dim <= MAX_HEAD_DIM:

@@ -487,10 +487,10 @@ def test_attention_refuses_what_it_cannot_take():
     table = torch.zeros(1, 2, dtype=torch.int32, device=DEV)
     with pytest.raises(ops.KernelError, match="groups"):
         ops.attention(q, 64, pool, pool, table, batch, torch.empty_like(q), 4, 3, 16, None, 0.25, kind=1)
-    big = torch.zeros(1, 528, device=DEV)
-    pool = torch.zeros(2, 1, 16, 528, device=DEV)
-    with pytest.raises(ops.KernelError, match="head size 528 is outside 1..512"):
-        ops.attention(big, 528, pool, pool.transpose(2, 3).contiguous(), table, batch, torch.empty_like(big), 1, 1, 528, None, 0.1, kind=1)
+    big = torch.zeros(1, 656, device=DEV)
+    pool = torch.zeros(2, 1, 16, 656, device=DEV)
+    with pytest.raises(ops.KernelError, match="head size 656 is outside 1..640"):
+        ops.attention(big, 656, pool, pool.transpose(2, 3).contiguous(), table, batch, torch.empty_like(big), 1, 1, 656, None, 0.1, kind=1)
 
 
 @pytest.mark.parametrize("dtype,kind", [(torch.bfloat16, 0), (torch.float32, 1)])

@@ -301,13 +301,13 @@ def latent_part(hidden, m, eps):
 LATENTS = [(3, 10, 6, 14, 9, 20, VH.rot(6, 30.0), 8), (4, 16, 16, 32, 64, 48, VH.rot(16, 1000.0, (8.0, 1.0, 4.0, 64.0)), 16),
            (20, 8, 24, 8, 40, 112, VH.rot(24, 100.0), 4), (2, 24, 0, 16, 16, 32, VH.rot(0, 10.0), 8), (6, 40, 32, 24, 24, 96, VH.rot(32, 500.0), 16),
            (2, 8, 8, 24, 1, 1, VH.rot(8, 20.0), 8), (6, 64, 32, 64, 96, 160, VH.rot(32, 10000.0), 16), (4, 16, 16, 16, 32, 240, VH.rot(16, 100.0), 12),
-           (1, 16, 64, 16, 48, 400, VH.rot(64, 100.0), 8)]
+           (1, 16, 64, 16, 48, 400, VH.rot(64, 100.0), 8), (5, 24, 64, 40, 56, 512, VH.rot(64, 1000.0), 16)]
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("heads,dim,rot_dim,vdim,q_rank,kv_rank,turn,page", LATENTS)
 def test_latent_attention_alone_in_portions(dtype, heads, dim, rot_dim, vdim, q_rank, kv_rank, turn, page):
-    """Query latents, halves that turn, sinks and gates; keys of 9 to 464 numbers, padded and not."""
+    """Query latents, halves that turn, sinks and gates; keys of 9 to 576 numbers, padded and not."""
     hidden, eps = 40, 1e-5
     m = VH.latent(heads, dim, rot_dim, vdim, q_rank, kv_rank, 1.2 / np.sqrt(dim + rot_dim), turn)["mixer"]
     rng = np.random.default_rng(heads * 10 + kv_rank)
@@ -365,7 +365,8 @@ def difference_part(hidden, m, eps):
 
 DIFFERENCES = [(6, 3, 6, 10, 4, 7, 8), (2, 2, 12, 5, 0, None, 8), (4, 1, 16, 32, 8, 24, 16), (3, 1, 5, 18, 2, 1, 4), (4, 2, 32, 64, 32, 100, 16),
                (6, 1, 40, 80, 20, 129, 16), (2, 1, 64, 128, 64, None, 16), (2, 1, 64, 64, 16, 300, 24), (10, 1, 32, 16, 16, 65, 8),
-               (2, 2, 80, 40, 80, 50, 8), (1, 1, 8, 200, 8, 33, 12), (2, 1, 72, 128, 8, None, 12)]
+               (2, 2, 80, 40, 80, 50, 8), (1, 1, 8, 200, 8, 33, 12), (2, 1, 72, 128, 8, None, 12),
+               (1, 1, 40, 530, 16, 70, 16)]
 
 
 @pytest.mark.parametrize("dtype", DTYPES)

@@ -67,9 +67,9 @@ def test_sizes_that_are_refused():
     for kind, good, bads in (
             ("mlstm", dict(hidden=8, heads=2, dim=4, vdim=4, gate_cap=5.0, eps=1e-5), (dict(gate_cap=0.0), dict(vdim=0), dict(dim=8000))),
             ("differential_attention", dict(hidden=8, heads=2, kv_heads=1, dim=4, vdim=4, scale=1.0, diff=0.1, eps=1e-5, position=none),
-             (dict(kv_heads=3), dict(window=0), dict(dim=300), dict(position=make_part("position", "rotary_interleaved", rotary_dim=4, theta=9.0)))),
+             (dict(kv_heads=3), dict(window=0), dict(dim=330), dict(position=make_part("position", "rotary_interleaved", rotary_dim=4, theta=9.0)))),
             ("latent_attention", dict(hidden=8, heads=2, dim=4, rot_dim=4, vdim=4, kv_rank=8, scale=1.0, eps=1e-5, position=none),
-             (dict(q_rank=0), dict(kv_rank=0), dict(kv_rank=600), dict(position=make_part("position", "rotary_neox", head_dim=8, theta=9.0))))):
+             (dict(q_rank=0), dict(kv_rank=0), dict(kv_rank=700), dict(position=make_part("position", "rotary_neox", head_dim=8, theta=9.0))))):
         make_part("mixer", kind, **good)
         for bad in bads:
             with pytest.raises(ConfigError):
